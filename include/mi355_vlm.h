@@ -544,7 +544,7 @@ int mi355_router_logits(int64_t tokens, int E, int K, const float* x, int64_t ld
 /* Grouped sigmoid router: s = sigmoid(logits), choice = s + correction (may be NULL); a group (E / groups neighbours) scores the sum of its two
  * largest choices, experts outside the `keep` best groups are excluded, the `top` largest choices win; wts = s / (sum + 1e-20) * scale.
  * ids int32 [tokens, top] in descending order of choice, wts fp32 [tokens, top].  mode 1 (softmax router): s = softmax(logits) over all experts, the `top`
- * largest win, wts = their s * scale without renormalisation (correction / groups unused).  mode 2: as mode 1 on logits + correction (a bias), the winners'
+ * largest win, wts = their s * scale without renormalisation (correction unused; a group scores its largest s).  mode 2: as mode 1 on logits + correction (a bias), the winners'
  * s divided by their sum, i.e. the softmax over the chosen logits alone, times scale. */
 int mi355_moe_route(int64_t tokens, int E, int top, int groups, int keep, const float* logits, const float* correction, float scale, int mode, int* ids,
                     float* wts, void* stream);
@@ -561,7 +561,7 @@ int mi355_bgemm(int batch, int M, int N, int K, const void* A, int a_dt, int64_t
                 const float* row_scale, int epi, int use_mfma, const float* bias, float limit, int n_out, void* stream);
 /* Causal attention with two-part keys over ragged batches: sequence s has n_new[s] query rows starting at row q_row0[s], `past[s]` earlier keys;
  * key j of it is K1 row k1_row0[s] + j (head stride k1_hs, D1 wide), K2 row k2_row0[s] + j (shared by heads, D2 wide), value row v_row0[s] + j.
- * Q fp32 [.., H, D1 + D2]; K1 / K2 / V / O of dtype dt.  A tile covers 32 / hm tokens x hm heads (hm > 1 needs k1_hs == v_hs == 0); the MFMA path (bf16,
+ * Q fp32 [.., H, D1 + D2]; K1 / K2 / V of dtype dt.  A tile covers 32 / hm tokens x hm heads (hm > 1 needs k1_hs == v_hs == 0); the MFMA path (bf16,
  * D1 + D2 <= 320, DV <= 256) 128 / hm tokens, and with splits > 1 deals a tile's keys to that many workgroups whose partial results meet in ws
  * (n_seq * head tiles * token tiles * splits * 128 * (2 + DV rounded up to 32 / 64 / 128 / 256) floats).  Under a plain window (keep_first == 0) the shares start
  * at the window's lower edge, and pooled rows (below) are part of what is dealt out.
@@ -571,12 +571,14 @@ int mi355_bgemm(int batch, int M, int N, int K, const void* A, int a_dt, int64_t
  * pool > 0 (needs window > 0, keep_first == 0, D2 == 0): besides the window the query at position i sees one pooled key / value row for every block b of
  * `pool` tokens with (b + 1) * pool <= i - window + 1; block b of sequence s is row pool_row0[s] + b of PK / PV (pitch ldp, head strides k1_hs / v_hs,
  * dtype dt); pooled rows and tokens share one softmax.  chunk > 0: positions are cut into chunks of that many, counted from the sequence's first token,
- * and a query sees only the keys j <= i of its own chunk, floor(j / chunk) == floor(i / chunk) (no kept first tokens, no pooled blocks). */
+ * and a query sees only the keys j <= i of its own chunk, floor(j / chunk) == floor(i / chunk) (no kept first tokens, no pooled blocks).
+ * sig_bias (fp32 [H], may be NULL): no softmax -- a visible key's weight is sigmoid(score + sig_bias[h]), not normalised (no softcap, no sink).  o_dt: dtype
+ * of the output rows O (fp32 also with bf16 keys and values). */
 int mi355_latent_attn(int n_seq, int max_new, int H, int hm, int D1, int D2, int DV, const float* Q, int64_t ldq, int q_hs, const void* K1, int64_t ldk1,
                       int k1_hs, const void* K2, int64_t ldk2, const void* V, int64_t ldv, int v_hs, void* O, int64_t ldo, int o_hs, int dt,
                       const int* q_row0, const int* n_new, const int* past, const int* k1_row0, const int* k2_row0, const int* v_row0, float scale,
                       int use_mfma, int splits, float* ws, int64_t ws_floats, int kv_rep, int window, int keep_first, float softcap, const float* sink,
-                      int pool, const void* PK, const void* PV, int64_t ldp, const int* pool_row0, int chunk, void* stream);
+                      int pool, const void* PK, const void* PV, int64_t ldp, const int* pool_row0, int chunk, const float* sig_bias, int o_dt, void* stream);
 
 /* ---- parallel-sublayer hybrid decoders in ragged batches (csrc/seqrec.hip) ---- */
 /* v = x + y1[t] + sum_{p < parts} y2[t * parts + p] (fp32 rows; y1 / y2 of dtype y*_dt, may be NULL); x_out (may be NULL or x) <- v.  For each weight
@@ -595,11 +597,11 @@ int mi355_ragged_conv(int64_t tokens, int n_seq, int C, int taps, const void* x,
  * (weights qw / kw fp32 [d], NULL: none) and a rotation of their first `dims` entries (layout as mi355_rope_heads); query head h times qscale[h] (may be NULL)
  * goes to q_out fp32 [t, h * d]; key and value heads go to cache row dst_row[t] = [G x d | G x dv] of dtype c_dt.  qt_every > 0: the query at position p
  * is also multiplied by 1 + qt_coef * ln(floor((p + 1) / qt_every) + 1).  vmix (fp32 rows [G x dv], pitch ldvm, may be NULL): the cached value is
- * (1 - lam) v + lam * vmix[t]. */
+ * (1 - lam) v + lam * vmix[t].  v_heads > 0: that many value heads instead of G (rows [H x d | G x d | v_heads x dv], cache rows [G x d | v_heads x dv]). */
 int mi355_qkv_rows_append(int64_t tokens, int H, int G, int d, int dv, const void* src, int src_dt, int64_t ld_src, const float* bias, const float* qw,
                           const float* kw, float eps, const float* qscale, int dims, int layout, const float* freq, const int* pos, const int* dst_row,
                           float* q_out, int64_t ldq, void* cache, int c_dt, int64_t ldc, float qt_coef, int qt_every, const float* vmix, int64_t ldvm, float lam,
-                          void* stream);
+                          int v_heads, void* stream);
 /* Gated delta rule over the rows [seq_off[s], seq_off[s+1]) of each sequence, state[slot[s]] (fp32 [H, dk, dv]) read and written.  q / k rows [G * dk] (raw:
  * made unit vectors here, x / sqrt(sum x^2 + 1e-6), q also times qscale), v rows [H * dv]; value head h uses query / key head h / (H / G);
  * beta = sigmoid(b[t, h]), g = exp(-exp(A_log[h]) * softplus(a[t, h] + dt_bias[h])).  Per token: S <- g S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q.
@@ -651,9 +653,26 @@ int mi355_rglru_ragged(int n_seq, int C, int blocks, float decay_c, const float*
  * gate_first 1: g = o silu(gate), g / rms(g) * w. */
 int mi355_gated_groupnorm(int64_t tokens, int n, int groups, const float* o, int64_t ldo_in, const float* w, const void* gate, int g_dt, int64_t ldg, int gate_first,
                           float eps, void* out, int out_dt, int64_t ldo, void* stream);
-/* Rows [n] -> [n].  kind 0: relu(x)^2; 1: tanh(x); 2: x[r, i] * sigmoid(gate[r, i / group]) (one gate per run of `group` entries). */
-int mi355_unary_rows(int64_t rows, int n, const void* x, int x_dt, int64_t ldx, int kind, const void* gate, int g_dt, int64_t ldg, int group, void* out,
+/* Rows [n] -> [n].  kind 0: relu(x)^2; 1: tanh(x); 2: x[r, i] * sigmoid(gate[r, i / group]) (one gate per run of `group` entries); 3: limit * tanh(x / limit). */
+int mi355_unary_rows(int64_t rows, int n, const void* x, int x_dt, int64_t ldx, int kind, const void* gate, int g_dt, int64_t ldg, int group, float limit, void* out,
                      int out_dt, int64_t ldo, void* stream);
+/* Minimal gated recurrence, per channel: z = sigmoid(zr[t, c]), u = x[t, c], candidate u + 1/2 (u >= 0) or sigmoid(u) (u < 0); S <- (1 - z) S + z * candidate;
+ * out[t, c] = S silu(g[t, c]).  zr, x fp32 rows (biases already added), g of dtype g_dt; state fp32 [slots, C], read and written at slot[s]. */
+int mi355_mingru_ragged(int n_seq, int C, const float* zr, int64_t ldz, const float* x, int64_t ldx, const void* g, int g_dt, int64_t ldg, const int* seq_off,
+                        const int* slot, float* state, void* out, int out_dt, int64_t ldo, void* stream);
+
+/* ---- decoders with parallel sublayers and a depth average in ragged batches (csrc/seqdep.hip) ---- */
+/* The sum, the depth average and the next norm of a block: v = x[t] + ls1 * (ca * ya[t] + cb * yb[t]) + ls2 * sum_{p < parts} y2[t * parts + p] (ya / yb / y2 may
+ * be NULL; ls1 / ls2 fp32 [width], NULL: 1); hist (fp32 [>= n_hist + 1, tokens, width], pitch hist_stride between results): result n_hist <- v;
+ * xa = sum_{j < n_hist} d[j] hist[j][t] + d[n_hist] v (d fp32 [n_hist + 1]; d NULL: xa = v, hist may then be NULL); x_out (may be NULL or x) <- xa;
+ * out (dtype out_dt) and out32 (fp32), each may be NULL <- xa / sqrt(mean(xa^2) + eps) * w (w fp32 [width], NULL: no norm).  width <= 16384. */
+int mi355_depth_sum(int64_t tokens, int width, const float* x, const void* ya, int ya_dt, int64_t ldya, float ca, const void* yb, int yb_dt, int64_t ldyb, float cb,
+                    const float* ls1, const void* y2, int y2_dt, int64_t ldy2, int parts, const float* ls2, float* hist, int64_t hist_stride, int n_hist,
+                    const float* d, float* x_out, const float* w, float eps, void* out, int out_dt, float* out32, void* stream);
+/* Join of differential attention: per head of D entries o = a1 - lam * a2 (fp32 rows [H x D]), o / sqrt(mean(o^2) + eps) * c, times sigmoid(gate) element by
+ * element (gate rows [H x D] of dtype g_dt, may be NULL). */
+int mi355_diff_join(int64_t tokens, int H, int D, const float* a1, int64_t lda1, const float* a2, int64_t lda2, float lam, float eps, float c, const void* gate, int g_dt,
+                    int64_t ldg, void* out, int out_dt, int64_t ldo, void* stream);
 
 #ifdef __cplusplus
 }

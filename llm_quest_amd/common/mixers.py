@@ -15,10 +15,15 @@
 * ``RecurrentGatedUnit``    -- a GELU branch times a real-gated linear recurrent unit behind a short convolution, block-diagonal gates, state in fp32;
 * ``StateSpaceDuality``     -- a selective state-space layer with one decay per head and token, a matrix state per head in fp32, gate before a grouped norm;
 * ``DecayBonusAttention``   -- token-shifted linear attention with a data-dependent decay per key channel and a bonus for the current token;
-* ``Relu2MLP``              -- an un-gated feed-forward around the squared ReLU.
-``LatentAttention`` also runs without a query latent, with rotate-half rotary, a sliding window and a sigmoid output gate; ``SlidingWindowAttention`` also
+* ``Relu2MLP``              -- an un-gated feed-forward around the squared ReLU;
+* ``DifferentialAttention`` -- two softmax maps per head over the same values, their weighted difference to unit RMS per head, a sigmoid gate per channel,
+  optionally on another layer's keys and values;
+* ``MinGatedUnit``          -- a minimal gated recurrence whose gate reads the current token only, state in fp32;
+* ``GroupedSoftmaxMoE``     -- softmax-scored squared-ReLU experts chosen inside the groups with the largest members, weights not renormalised.
+``LatentAttention`` also runs without a query latent, without a rotated part, with rotate-half rotary, a sliding window, a sink in the denominator and a sigmoid output
+gate (per channel or per head); ``SlidingWindowAttention`` also
 with capped scores, a position-dependent query temperature, pooled blocks before the window, a sink in the denominator, value mixing between layers,
-chunks instead of a window, rescaled rotary frequencies and one sigmoid output gate per head; ``SoftmaxTopkMoE`` also with a router bias, weights that are the
+chunks instead of a window, rescaled rotary frequencies, one sigmoid output gate per head and sigmoid weights without a softmax; ``SoftmaxTopkMoE`` also with a router bias, weights that are the
 softmax over the winners alone, SiLU-gated experts and a shared expert.
 
 They run one *step* of a batch (``SeqStep``): the new tokens of every sequence, packed row after row, against what ``utils.SlotStateCache`` holds.  Inference
@@ -114,21 +119,24 @@ class LatentAttention(_Frozen):
     ``kv_rank``.  ``kv_from``: read that layer's cached rows instead of projecting own ones.  Rotary: ``rot_dims`` of the rotated part turn (base
     ``rot_base``), as interleaved pairs or -- ``rot_layout`` 1 -- entry i with entry i + rot_dims / 2.  ``q_rank`` 0: the query is projected from the
     input directly, without a latent.  ``window`` > 0: position i sees the keys j with 0 <= i - j < window.  ``gate``: the concatenated heads are multiplied
-    by the sigmoid of a projection of the mixer's input before the output projection."""
+    by the sigmoid of a projection of the mixer's input before the output projection -- element by element (True) or one number per head ("head").
+    ``sink``: a learned number per head whose exponential joins the softmax denominator.  ``rot_dim`` may be 0 (no positions)."""
 
-    def __init__(self, width, heads, dim, rot_dim, vdim, q_rank, kv_rank, scale, rot_dims, rot_base, eps, layer_idx, kv_from=None, rot_layout=0, window=0, gate=False):
+    def __init__(self, width, heads, dim, rot_dim, vdim, q_rank, kv_rank, scale, rot_dims, rot_base, eps, layer_idx, kv_from=None, rot_layout=0, window=0, gate=False,
+                 sink=False):
         super().__init__()
         self.width, self.heads, self.dim, self.rot_dim, self.vdim = width, heads, dim, rot_dim, vdim
         self.q_rank, self.kv_rank, self.scale, self.rot_dims, self.rot_base, self.eps = q_rank, kv_rank, float(scale), rot_dims, float(rot_base), float(eps)
         self.layer_idx, self.kv_from = layer_idx, kv_from
-        self.rot_layout, self.window, self.gate = int(rot_layout), int(window), bool(gate)
+        self.rot_layout, self.window, self.gate = int(rot_layout), int(window), gate
         if rot_dims % 2 or rot_dims > rot_dim:
             raise ValueError("LatentAttention: the rotated entries are an even number <= rot_dim")
         own = kv_from is None
         # projections of the input side by side -> one product: [query latent, or the queries themselves | kv_rank + rot_dim | gate]
         self.q_cols = q_rank if q_rank else heads * (dim + rot_dim)
         self.kv_cols = kv_rank + rot_dim if own else 0
-        self.w_down = self._param(self.q_cols + self.kv_cols + (heads * vdim if gate else 0), width)
+        self.w_down = self._param(self.q_cols + self.kv_cols + (heads if gate == "head" else heads * vdim if gate else 0), width)
+        self.sink = self._param(heads) if sink else None
         self.q_norm = self._param(q_rank) if q_rank else None
         self.kv_norm = self._param(kv_rank) if own else None
         self.w_uq = self._param(heads * (dim + rot_dim), q_rank) if q_rank else None
@@ -143,6 +151,7 @@ class LatentAttention(_Frozen):
         if self._ready != device:
             self.q_norm32 = _f32(self.q_norm)
             self.kv_norm32 = _f32(self.kv_norm)
+            self.sink32 = _f32(self.sink)
             self.freq = S.rope_frequencies(self.rot_dims, self.rot_base, device)
             self._ready = device
 
@@ -155,9 +164,12 @@ class LatentAttention(_Frozen):
         src = self.layer_idx if own else self.kv_from
         cache2d = st.cache.rows2d(self.layer_idx)
         lay, win = self.rot_layout, self.window
-        # without a query latent the projection feeds fp32 work only (rotary, the latent's norm, the gate's sigmoid): it leaves the product as fp32
-        down = S.linear(h, self.w_down, out_dtype=None if self.q_rank else F32)
-        q = S.linear(S.rmsnorm_rows(down[:, :Rq], self.q_norm32, self.eps), self.w_uq) if self.q_rank else down[:, :Rq]
+        # without a query latent the projection feeds fp32 work only (rotary, the latent's norm, the gate's sigmoid): it leaves the product as fp32; so it
+        # does where the gate's number per head is a column of it
+        down = S.linear(h, self.w_down, out_dtype=None if self.q_rank and self.gate != "head" else F32)
+        # prompts without a rotated part take the queries as the product leaves them (fp32, what the attention reads)
+        plain = st.fresh and not dr
+        q = S.linear(S.rmsnorm_rows(down[:, :Rq], self.q_norm32, self.eps, out_dtype=h.dtype), self.w_uq, out_dtype=F32 if plain else None) if self.q_rank else down[:, :Rq]
         kv_src = down[:, Rq : Rq + self.kv_cols]
         if own:
             S.latent_kv_append(kv_src, R, dr, self.kv_norm32, self.eps, st.pos, st.dst_row, self.freq, self.rot_dims, cache2d, layout=lay)
@@ -170,27 +182,32 @@ class LatentAttention(_Frozen):
                 st.local[src] = lat
             lat = st.local[src]
             kv = S.linear(lat[:, :R], self.w_ukv)  # [T, H*dn | H*dv]
-            q32 = torch.empty((T, H * (dn + dr)), dtype=F32, device=h.device)
-            S.rope_heads(q, H, dn + dr, dn + dr, 0, q32, dn + dr, 0, dn, self.rot_dims, self.freq, st.pos, layout=lay)
+            q32 = q
+            if not plain:
+                q32 = torch.empty((T, H * (dn + dr)), dtype=F32, device=h.device)
+                S.rope_heads(q, H, dn + dr, dn + dr, 0, q32, dn + dr, 0, dn, self.rot_dims, self.freq, st.pos, layout=lay)
             ctx = torch.empty((T, H * dv), dtype=st.act_dtype, device=h.device)
-            S.latent_attn(q32, kv[:, : H * dn], lat[:, R:], kv[:, H * dn :], ctx, H, 1, dn, dr, dv, dn + dr, dn, dv, dv,
-                          (st.q_row0, st.n_new, st.past, st.q_row0, st.q_row0, st.q_row0), st.max_new, self.scale, window=win)
+            S.latent_attn(q32, kv[:, : H * dn], lat[:, R:] if dr else None, kv[:, H * dn :], ctx, H, 1, dn, dr, dv, dn + dr, dn, dv, dv,
+                          (st.q_row0, st.n_new, st.past, st.q_row0, st.q_row0, st.q_row0), st.max_new, self.scale, window=win, sink=self.sink32)
         else:
             # continuation: the key up-projection folded onto the query, the value up-projection applied after the attention -- the cache rows are
             # keys and values of every head as they stand
             qf = torch.empty((T, H * (R + dr)), dtype=F32, device=h.device)
             S.bgemm(q, self.w_ukv, qf, T, R, dn, batch=H, lda=q.stride(0), a_bs=dn + dr, sbn=1, sbk=R, b_bs=dn * R, ldc=H * (R + dr), c_bs=R + dr)
-            S.rope_heads(q, H, dr, dn + dr, dn, qf, R + dr, R, 0, self.rot_dims, self.freq, st.pos, layout=lay)
+            if dr:
+                S.rope_heads(q, H, dr, dn + dr, dn, qf, R + dr, R, 0, self.rot_dims, self.freq, st.pos, layout=lay)
             hm = 1
             while hm < min(H, 32):
                 hm *= 2
             ol = torch.empty((T, H * R), dtype=st.act_dtype, device=h.device)
             for v0 in range(0, R, 512):  # the attention takes values up to 512 wide: a wider latent goes in parts (the scores are the same every time)
-                S.latent_attn(qf, cache2d, cache2d[:, R:], cache2d[:, v0:], ol[:, v0:], H, hm, R, dr, min(512, R - v0), R + dr, 0, 0, R,
-                              (st.q_row0, st.n_new, st.past, st.cache_row0, st.cache_row0, st.cache_row0), st.max_new, self.scale, max_keys=st.max_keys, window=win)
+                S.latent_attn(qf, cache2d, cache2d[:, R:] if dr else None, cache2d[:, v0:], ol[:, v0:], H, hm, R, dr, min(512, R - v0), R + dr, 0, 0, R,
+                              (st.q_row0, st.n_new, st.past, st.cache_row0, st.cache_row0, st.cache_row0), st.max_new, self.scale, max_keys=st.max_keys, window=win, sink=self.sink32)
             ctx = torch.empty((T, H * dv), dtype=st.act_dtype, device=h.device)
             S.bgemm(ol, self.w_ukv[H * dn :], ctx, T, dv, R, batch=H, lda=H * R, a_bs=R, sbn=R, sbk=1, b_bs=dv * R, ldc=H * dv, c_bs=dv)
-        if self.gate:
+        if self.gate == "head":
+            ctx = S.unary_rows(ctx, S.UNARY_HEAD_GATE, gate=down[:, Rq + self.kv_cols :], group=dv)
+        elif self.gate:
             ctx = S.act_rows(ctx, S.ACT_SIGMOID_GATE, gate=down[:, Rq + self.kv_cols :])
         return S.linear(ctx, self.w_o, out_dtype=out_dtype)
 
@@ -250,19 +267,33 @@ class GroupedSigmoidMoE(_Frozen):
             self.correction32 = _f32(self.correction)
             self._ready = device
 
+    def route(self, logits):
+        return S.moe_route(logits, self.correction32, self.top, self.groups, self.keep, self.scale)
+
     @torch.no_grad()
     def step(self, x32, h):
         """x32: the fp32 residual rows (the router reads them), h: the same rows in the activation dtype -> fp32 [T * top, width]."""
         self.prepare(h.device)
         T, E, top = h.shape[0], self.experts, self.top
         logits = S.router_logits(x32, self.w_router)
-        ids, wts = S.moe_route(logits, self.correction32, top, self.groups, self.keep, self.scale)
+        ids, wts = self.route(logits)
         offs, perm = S.moe_dispatch(ids.view(-1), E)
         act = torch.empty((T * top, self.ff), dtype=h.dtype, device=h.device)
         S.bgemm(h, self.w_up, act, T * top, self.ff, self.width, batch=E, sbn=self.width, b_bs=self.ff * self.width, grp_offs=offs, a_rows=perm, a_div=top, epi=1)
         out = torch.empty((T * top, self.width), dtype=F32, device=h.device)
         S.bgemm(act, self.w_down, out, T * top, self.width, self.ff, batch=E, sbn=self.ff, b_bs=self.width * self.ff, grp_offs=offs, c_rows=perm, row_scale=wts.view(-1))
         return out
+
+
+class GroupedSoftmaxMoE(GroupedSigmoidMoE):
+    """The same squared-ReLU experts behind a softmax router: scores are the softmax over ALL experts, a group scores its largest member, the ``top`` largest
+    scores inside the ``keep`` best groups win and ARE the weights (times ``scale``, not renormalised)."""
+
+    def __init__(self, width, ff, experts, top, groups=1, keep=1, scale=1.0):
+        super().__init__(width, ff, experts, top, groups, keep, scale, correction=False)
+
+    def route(self, logits):
+        return S.moe_route(logits, None, self.top, self.groups, self.keep, self.scale, softmax=True)
 
 
 # ----------------------------------------------------------------------------------------------- mechanisms of parallel-sublayer hybrid decoders
@@ -355,11 +386,13 @@ class SlidingWindowAttention(_Frozen):
         frequencies for a longer context (``kernels_seq.scaled_rope_frequencies``);
       * ``head_gate``        -- head h's output is multiplied by sigmoid(w_g h)_h, one number per head from the mixer's input, before the output projection
         (its rows follow the value rows in ``w_qkv``);
-      * ``o_bias``           -- whether the output projection has a bias (default: as ``bias``).
+      * ``o_bias``           -- whether the output projection has a bias (default: as ``bias``);
+      * ``sigmoid``          -- no softmax: the weight of a visible key is sigmoid(score + pb[h]), ``pb`` a learned number per head, weights not normalised.
     ``step(..., proj=rows)``: the caller has already taken the input product (with its biases) -- a mixer beside this one shares it."""
 
     def __init__(self, width, heads, kv_heads, dim, vdim, scale, window, keep_first, rot_dims, rot_base, eps, layer_idx, qk_norm=True, bias=True, temp=True,
-                 softcap=0.0, q_temp=None, pool=0, sink=False, v_mix=None, chunk=0, rot_layout=0, rot_scaling=None, head_gate=False, o_bias=None):
+                 softcap=0.0, q_temp=None, pool=0, sink=False, v_mix=None, chunk=0, rot_layout=0, rot_scaling=None, head_gate=False, o_bias=None,
+                 sigmoid=False):
         super().__init__()
         if heads % kv_heads:
             raise ValueError("SlidingWindowAttention: heads must be a multiple of kv_heads")
@@ -371,6 +404,8 @@ class SlidingWindowAttention(_Frozen):
             raise ValueError("SlidingWindowAttention: v_mix is None, 'first' or 'mix'")
         if chunk and (window or keep_first or pool):
             raise ValueError("SlidingWindowAttention: chunks stand instead of a window (no kept first tokens, no pooled blocks)")
+        if sigmoid and (softcap or sink):
+            raise ValueError("SlidingWindowAttention: sigmoid weights have neither a cap nor a denominator")
         self.chunk, self.rot_layout, self.rot_scaling, self.head_gate = int(chunk or 0), int(rot_layout), dict(rot_scaling) if rot_scaling else None, bool(head_gate)
         self.width, self.heads, self.kv_heads, self.dim, self.vdim, self.scale, self.window, self.keep_first = width, heads, kv_heads, dim, vdim, float(scale), int(window), int(keep_first)
         self.rot_dims, self.rot_base, self.eps, self.layer_idx = rot_dims, float(rot_base), float(eps), layer_idx
@@ -383,6 +418,7 @@ class SlidingWindowAttention(_Frozen):
         self.k_norm = self._param(dim) if qk_norm else None
         self.temp = self._param(heads) if temp else None
         self.sink = self._param(heads) if sink else None
+        self.pb = self._param(heads) if sigmoid else None
         self.lam = self._param(1) if v_mix == "mix" else None
         self.w_o = self._param(width, heads * vdim)
         self.b_o = self._param(width) if (bias if o_bias is None else o_bias) else None
@@ -406,6 +442,7 @@ class SlidingWindowAttention(_Frozen):
     def prepare(self, device):
         if self._ready != device:
             self.b_qkv32, self.q_norm32, self.k_norm32, self.b_o32, self.sink32 = _f32(self.b_qkv), _f32(self.q_norm), _f32(self.k_norm), _f32(self.b_o), _f32(self.sink)
+            self.pb32 = _f32(self.pb)
             t = _f32(self.temp) if self.temp is not None else torch.ones(self.heads, dtype=F32, device=device)
             # the score's factors: folded onto the query, unless the scaled score goes through the cap (then the kernel scales)
             self.qscale = None if self.softcap else (t * self.scale).contiguous()
@@ -447,7 +484,7 @@ class SlidingWindowAttention(_Frozen):
         hm = _largest_pow2_divisor(H // G)
         S.latent_attn(q, cache2d, None, cache2d[:, G * d :], ctx, H, hm, d, 0, dv, d, d, dv, dv, (st.q_row0, st.n_new, st.past, st.cache_row0, st.cache_row0, st.cache_row0),
                       st.max_new, self.scale if self.softcap else 1.0, max_keys=st.max_keys, kv_rep=H // G, window=self.window, keep_first=self.keep_first,
-                      softcap=self.softcap, sink=self.sink32, pool=self.pool, pooled=pooled, pool_row0=row0, chunk=self.chunk)
+                      softcap=self.softcap, sink=self.sink32, pool=self.pool, pooled=pooled, pool_row0=row0, chunk=self.chunk, sig_bias=self.pb32)
         if self.head_gate:
             ctx = S.unary_rows(ctx, S.UNARY_HEAD_GATE, gate=gate, group=dv)
         return S.linear(ctx, self.w_o, bias=self.b_o32, out_dtype=out_dtype)
@@ -802,3 +839,97 @@ class Relu2MLP(_Frozen):
     @torch.no_grad()
     def step(self, h, out_dtype=None):
         return S.linear(S.unary_rows(S.linear(h, self.w_up), S.UNARY_RELU2), self.w_down, out_dtype=out_dtype)
+
+
+# ----------------------------------------------------------------------------------------------- mechanisms of decoders with parallel sublayers and a depth average
+class DifferentialAttention(_Frozen):
+    """Differential attention: per head two softmax maps (queries and keys of ``dim`` each, laid out head by head as [map 1, map 2]) over the same values
+    [``vdim``], grouped queries, biases on q / k / v.  o = a1 - lambda a2 with lambda = exp(lq1 . lk1) - exp(lq2 . lk2) + ``diff``, one number for the layer;
+    every head's o is divided by its root mean square, times 1 - ``diff``; with ``gate`` the concatenated heads are multiplied by the sigmoid of a projection of
+    the mixer's input; output projection.  Rotary on the first ``rot_dims`` entries of each map (``rot_layout`` as elsewhere).  ``kv_from``: the layer reads that
+    layer's cached keys and values and projects queries only.  Keys and values are cached token-major, [kv_heads x 2 dim | kv_heads x vdim] per row."""
+
+    def __init__(self, width, heads, kv_heads, dim, vdim, scale, diff, rot_dims, rot_base, eps, layer_idx, kv_from=None, rot_layout=0, bias=True, gate=True):
+        super().__init__()
+        if heads % kv_heads:
+            raise ValueError("DifferentialAttention: heads must be a multiple of kv_heads")
+        if rot_dims % 2 or rot_dims > dim:
+            raise ValueError("DifferentialAttention: the rotated entries are an even number <= dim")
+        self.width, self.heads, self.kv_heads, self.dim, self.vdim, self.scale, self.diff = width, heads, kv_heads, dim, vdim, float(scale), float(diff)
+        self.rot_dims, self.rot_base, self.eps, self.layer_idx, self.kv_from, self.rot_layout = rot_dims, float(rot_base), float(eps), layer_idx, kv_from, int(rot_layout)
+        self.q_cols = 2 * heads * dim
+        self.kv_cols = kv_heads * (2 * dim + vdim) if kv_from is None else 0
+        n = self.q_cols + self.kv_cols
+        self.w_in = self._param(n + (heads * vdim if gate else 0), width)  # [q | k | v | gate] rows -> one product
+        self.b_in = self._param(n) if bias else None
+        self.lq1, self.lk1, self.lq2, self.lk2 = self._param(dim), self._param(dim), self._param(dim), self._param(dim)
+        self.gate = bool(gate)
+        self.w_o = self._param(width, heads * vdim)
+        self._ready = None
+
+    def cache_spec(self):
+        return {"rows": self.kv_cols, "states": {}} if self.kv_from is None else ("shared", self.kv_from)
+
+    def prepare(self, device):
+        if self._ready != device:
+            b = _f32(self.b_in)
+            self.b_in32 = None if b is None else torch.cat([b, b.new_zeros(self.w_in.shape[0] - b.numel())]).contiguous()
+            self.freq = S.rope_frequencies(self.rot_dims, self.rot_base, device) if self.rot_dims else None
+            dot = lambda a, c: float((a.double() * c.double()).sum().exp().item())
+            self.lam = dot(self.lq1, self.lk1) - dot(self.lq2, self.lk2) + self.diff
+            self._ready = device
+
+    @torch.no_grad()
+    def step(self, h, st, out_dtype=None):
+        self.prepare(h.device)
+        H, G, d, dv = self.heads, self.kv_heads, self.dim, self.vdim
+        T, n = h.shape[0], self.q_cols + self.kv_cols
+        cache2d = st.cache.rows2d(self.layer_idx)
+        proj = S.linear(h, self.w_in, out_dtype=F32, bias=self.b_in32)
+        if self.kv_from is None:
+            q = S.qkv_rows_append(proj[:, :n], 2 * H, 2 * G, d, dv, None, None, None, self.eps, None, self.rot_dims, self.rot_layout, self.freq, st.pos, st.dst_row, cache2d,
+                                  v_heads=G)
+        else:
+            q = torch.empty((T, n), dtype=F32, device=h.device)
+            S.rope_heads(proj[:, :n], 2 * H, d, d, 0, q, d, 0, 0, self.rot_dims, self.freq, st.pos, layout=self.rot_layout)
+        maps = []
+        for m in (0, 1):  # the maps' outputs stay fp32: their difference is small where the maps agree
+            a = torch.empty((T, H * dv), dtype=F32, device=h.device)
+            S.latent_attn(q[:, m * d :], cache2d[:, m * d :], None, cache2d[:, 2 * G * d :], a, H, _largest_pow2_divisor(H // G), d, 0, dv, 2 * d, 2 * d, dv, dv,
+                          (st.q_row0, st.n_new, st.past, st.cache_row0, st.cache_row0, st.cache_row0), st.max_new, self.scale, max_keys=st.max_keys, kv_rep=H // G)
+            maps.append(a)
+        ctx = S.diff_join(maps[0], maps[1], H, dv, self.lam, self.eps, 1.0 - self.diff, proj[:, n:] if self.gate else None, st.act_dtype)
+        return S.linear(ctx, self.w_o, out_dtype=out_dtype)
+
+
+class MinGatedUnit(_Frozen):
+    """Minimal gated recurrence over ``channels``: z = sigmoid(W_z h + b), u = W_x h + b, candidate u + 1/2 where u >= 0 and sigmoid(u) where u < 0;
+    S <- (1 - z) S + z * candidate, carried per sequence in fp32 from zero; output W_o (S silu(W_g h))."""
+
+    in_weight = "w_in"
+
+    def __init__(self, width, channels, layer_idx, name="mg"):
+        super().__init__()
+        self.width, self.channels, self.layer_idx, self.name = width, channels, layer_idx, name
+        self.w_in = self._param(3 * channels, width)  # [z | x | gate] rows
+        self.b_in = self._param(2 * channels)
+        self.w_o = self._param(width, channels)
+        self._ready = None
+
+    def in_bias(self):
+        b = _f32(self.b_in)
+        return torch.cat([b, b.new_zeros(self.channels)])
+
+    def cache_spec(self):
+        return {"rows": None, "states": {self.name + "_S": (self.channels,)}}
+
+    @torch.no_grad()
+    def step(self, h, st, out_dtype=None, proj=None):
+        C = self.channels
+        if proj is None:
+            if self._ready != h.device:
+                self.b_in32 = self.in_bias()
+                self._ready = h.device
+            proj = S.linear(h, self.w_in, out_dtype=F32, bias=self.b_in32)
+        mix = S.mingru(proj[:, :C], proj[:, C : 2 * C], proj[:, 2 * C :], st.seq_off, st.slots, st.cache.state(self.layer_idx, self.name + "_S"), st.act_dtype)
+        return S.linear(mix, self.w_o, out_dtype=out_dtype)

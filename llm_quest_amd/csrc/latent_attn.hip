@@ -9,7 +9,8 @@
 // (window, keep_first): key steps that no row of a tile can see are skipped.  Further options: tanh-capped scores (softcap), a per-head sink that
 // only enters the softmax denominator, and POOLED blocks in front of a window -- one mean key / value row per `pool` tokens, kept by the caller in a
 // second buffer; the query at position i sees block b iff all of its tokens have left the window, (b + 1) pool <= i - window + 1.  Pooled rows
-// and tokens share one softmax: the key loop simply runs over the pooled rows first.
+// and tokens share one softmax: the key loop simply runs over the pooled rows first.  Without a softmax (sig_bias): the weight of a visible key is
+// sigmoid(score + sig_bias[head]), not normalised -- no running maximum, no rescaling, no denominator.
 // Scores, softmax statistics and the output accumulators are fp32.  A tile is `tm` tokens x `hm` heads = 32 query rows (hm > 1 only with shared
 // keys and values) against 64 keys at a time.
 //
@@ -41,6 +42,8 @@ struct LatAttnArgs {
     const void *PK, *PV;
     int64_t ldp;
     const int* pool_row0;
+    const float* sig_bias;  // fp32 [H] or NULL: weights sigmoid(score + sig_bias[head]) instead of a softmax
+    int o_dt;               // dtype of the output rows (MI355_DT_*)
 };
 
 // pooled blocks the query at position lim sees: those that end at or before lim - window
@@ -105,6 +108,11 @@ __global__ __launch_bounds__(256) void latent_attn_fma_kernel(LatAttnArgs p) {
     int npv[2];
 #pragma unroll
     for (int a = 0; a < 2; ++a) npv[a] = p.pool > 0 ? pooled_visible(lim[a], p.window, p.pool) : 0;
+    float sb[2] = {0.f, 0.f};  // the rows' biases of the sigmoid weights
+    if (p.sig_bias) {
+#pragma unroll
+        for (int a = 0; a < 2; ++a) sb[a] = p.sig_bias[min(head0 + (2 * ty + a) % p.hm, p.H - 1)];
+    }
     for (int it = -pool_steps;; ++it) {
         const bool seg = it < 0;  // the pooled rows come first
         const int j0 = seg ? (it + pool_steps) * AN : it * AN;
@@ -160,11 +168,11 @@ __global__ __launch_bounds__(256) void latent_attn_fma_kernel(LatAttnArgs p) {
             for (int of = 8; of > 0; of >>= 1) mx = fmaxf(mx, __shfl_xor(mx, of, 64));
             const float m_new = fmaxf(m_run[a], mx);
             const float base = m_new == -__builtin_huge_valf() ? 0.f : m_new;
-            const float f = expf(m_run[a] - base);
+            const float f = p.sig_bias ? 1.0f : expf(m_run[a] - base);
             float sum = 0.f;
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
-                const float e = expf(acc[a][i] - base);
+                const float e = p.sig_bias ? 1.0f / (1.0f + expf(-(acc[a][i] + sb[a]))) : expf(acc[a][i] - base);  // a hidden key's -inf gives 0 either way
                 Ps[2 * ty + a][tx + 16 * i] = e;
                 sum += e;
             }
@@ -209,6 +217,7 @@ __global__ __launch_bounds__(256) void latent_attn_fma_kernel(LatAttnArgs p) {
                 f = expf(m_run[a] - m2);
                 l = l * f + expf(sk - m2);
             }
+            if (p.sig_bias) l = 1.0f;
             ls[r] = l, fs[r] = f;
         }
     }
@@ -224,7 +233,7 @@ __global__ __launch_bounds__(256) void latent_attn_fma_kernel(LatAttnArgs p) {
             const int col = c + 64 * i;
             if (col >= p.DV) continue;
             const float v = o[r][i] * inv;
-            if (p.dt == MI355_DT_F32) ((float*)p.O)[ob + col] = v;
+            if (p.o_dt == MI355_DT_F32) ((float*)p.O)[ob + col] = v;
             else ((bf16_t*)p.O)[ob + col] = f2bf(v);
         }
     }
@@ -238,7 +247,7 @@ __global__ __launch_bounds__(256) void latent_attn_fma_kernel(LatAttnArgs p) {
 // LDS as [64 keys][DKP] (main part and rotated part side by side, zero padded), the value tile transposed as [DVP][64 keys].
 #define MQ 128
 #define MKT 64
-template <int DKS, int NVB>
+template <int DKS, int NVB, bool SIG>
 __global__ __launch_bounds__(256) void latent_attn_mfma_kernel(LatAttnArgs p, int vec_ok) {
     constexpr int DKP = DKS * 8, DVP = NVB * 32, KLD = DKP + 4, VLD = MKT + 4;
     __shared__ __attribute__((aligned(16))) bf16_t Ks[MKT * KLD];
@@ -305,6 +314,7 @@ __global__ __launch_bounds__(256) void latent_attn_mfma_kernel(LatAttnArgs p, in
     const int npv = p.pool > 0 ? pooled_visible(lim, p.window, p.pool) : 0;  // the pooled rows this lane's query sees
     const int64_t pr0 = p.pool > 0 ? p.pool_row0[s] : 0;
     const float capl = p.softcap * 1.4426950408889634f;
+    const float sgb = SIG ? p.sig_bias[row_ok ? head : 0] * 1.4426950408889634f : 0.f;
     for (int v = v_lo; v < v_hi; ++v) {
         const bool seg = v < pool_steps;  // the pooled rows come first
         const int j0 = seg ? v * MKT : key_lo + (v - pool_steps) * MKT;
@@ -367,45 +377,64 @@ __global__ __launch_bounds__(256) void latent_attn_mfma_kernel(LatAttnArgs p, in
                 sacc[kb] = __builtin_amdgcn_mfma_f32_32x32x8bf16_1k(a, qf[st], sacc[kb], 0, 0, 0);
             }
         }
-        // ---- online softmax for the lane's query (keys kb * 32 + 8 g + 4 hf + i)
-        float mx = NEG;
-#pragma unroll
-        for (int kb = 0; kb < 2; ++kb)
-#pragma unroll
-            for (int r = 0; r < 16; ++r) {
-                const int j = j0 + kb * 32 + 8 * (r >> 2) + 4 * hf + (r & 3);
-                const bool vis = seg ? j < npv : (key_visible(j, lim, p.window, p.keep_first, p.chunk) && j < n_keys);
-                const float v = !vis ? NEG : (p.softcap > 0.f ? capl * tanhf(sacc[kb][r] * p.scale / p.softcap) : sacc[kb][r] * sc2);
-                sacc[kb][r] = v;
-                mx = fmaxf(mx, v);
-            }
-        mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
-        const float m_new = fmaxf(m_run, mx);
-        const float base = m_new == NEG ? 0.f : m_new;
-        const float f = exp2f(m_run - base);
-        float sum = 0.f;
+        // ---- weights of the lane's query (keys kb * 32 + 8 g + 4 hf + i)
         bf16x4 pf[8];
+        float f = 1.f;
+        if constexpr (SIG) {
 #pragma unroll
-        for (int kb = 0; kb < 2; ++kb)
+            for (int kb = 0; kb < 2; ++kb)
 #pragma unroll
-            for (int g = 0; g < 4; ++g) {
-                float e[4];
+                for (int g = 0; g < 4; ++g) {
+                    float e[4];
 #pragma unroll
-                for (int i = 0; i < 4; ++i) {
-                    e[i] = exp2f(sacc[kb][4 * g + i] - base);
-                    sum += e[i];
+                    for (int i = 0; i < 4; ++i) {
+                        const int j = j0 + kb * 32 + 8 * g + 4 * hf + i;
+                        const bool vis = seg ? j < npv : (key_visible(j, lim, p.window, p.keep_first, p.chunk) && j < n_keys);
+                        e[i] = vis ? __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-fmaf(sacc[kb][4 * g + i], sc2, sgb))) : 0.f;
+                    }
+                    u32x2 pk = {pack_bf2(e[0], e[1]), pack_bf2(e[2], e[3])};
+                    pf[kb * 4 + g] = __builtin_bit_cast(bf16x4, pk);
                 }
-                u32x2 pk = {pack_bf2(e[0], e[1]), pack_bf2(e[2], e[3])};
-                pf[kb * 4 + g] = __builtin_bit_cast(bf16x4, pk);
-            }
-        sum += __shfl_xor(sum, 32, 64);
-        l_run = l_run * f + sum;
-        m_run = m_new;
+        } else {  // online softmax
+            float mx = NEG;
+#pragma unroll
+            for (int kb = 0; kb < 2; ++kb)
+#pragma unroll
+                for (int r = 0; r < 16; ++r) {
+                    const int j = j0 + kb * 32 + 8 * (r >> 2) + 4 * hf + (r & 3);
+                    const bool vis = seg ? j < npv : (key_visible(j, lim, p.window, p.keep_first, p.chunk) && j < n_keys);
+                    const float v = !vis ? NEG : (p.softcap > 0.f ? capl * tanhf(sacc[kb][r] * p.scale / p.softcap) : sacc[kb][r] * sc2);
+                    sacc[kb][r] = v;
+                    mx = fmaxf(mx, v);
+                }
+            mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+            const float m_new = fmaxf(m_run, mx);
+            const float base = m_new == NEG ? 0.f : m_new;
+            f = exp2f(m_run - base);
+            float sum = 0.f;
+#pragma unroll
+            for (int kb = 0; kb < 2; ++kb)
+#pragma unroll
+                for (int g = 0; g < 4; ++g) {
+                    float e[4];
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) {
+                        e[i] = exp2f(sacc[kb][4 * g + i] - base);
+                        sum += e[i];
+                    }
+                    u32x2 pk = {pack_bf2(e[0], e[1]), pack_bf2(e[2], e[3])};
+                    pf[kb * 4 + g] = __builtin_bit_cast(bf16x4, pk);
+                }
+            sum += __shfl_xor(sum, 32, 64);
+            l_run = l_run * f + sum;
+            m_run = m_new;
+        }
         // ---- O^T <- O^T * f + V^T P^T
 #pragma unroll
         for (int vb = 0; vb < NVB; ++vb) {
 #pragma unroll
-            for (int i = 0; i < 16; ++i) oacc[vb][i] *= f;
+            for (int i = 0; i < 16; ++i)
+                if constexpr (!SIG) oacc[vb][i] *= f;
 #pragma unroll
             for (int ks = 0; ks < 8; ++ks) {
                 const bf16x4 a = *(const bf16x4*)&Vt[(vb * 32 + ln) * VLD + 8 * ks + 4 * hf];
@@ -424,12 +453,24 @@ __global__ __launch_bounds__(256) void latent_attn_mfma_kernel(LatAttnArgs p, in
         return;
     }
     if (!row_ok) return;
-    float inv = 1.0f / l_run;
-    if (p.sink) {  // the sink joins the denominator (statistics are in base-2 units)
+    float inv = SIG ? 1.0f : 1.0f / l_run;
+    if (!SIG && p.sink) {  // the sink joins the denominator (statistics are in base-2 units)
         const float sk = p.sink[head] * 1.4426950408889634f, m2 = fmaxf(m_run, sk), f = exp2f(m_run - m2);
         inv = f / (l_run * f + exp2f(sk - m2));
     }
-    bf16_t* orow = (bf16_t*)p.O + (qr0 + tok) * p.ldo + (int64_t)head * p.o_hs;
+    const int64_t o0 = (qr0 + tok) * p.ldo + (int64_t)head * p.o_hs;
+    if (p.o_dt == MI355_DT_F32) {
+        float* orow = (float*)p.O + o0;
+#pragma unroll
+        for (int vb = 0; vb < NVB; ++vb)
+#pragma unroll
+            for (int r = 0; r < 16; ++r) {
+                const int dv = vb * 32 + 8 * (r >> 2) + 4 * hf + (r & 3);
+                if (dv < p.DV) orow[dv] = oacc[vb][r] * inv;
+            }
+        return;
+    }
+    bf16_t* orow = (bf16_t*)p.O + o0;
 #pragma unroll
     for (int vb = 0; vb < NVB; ++vb)
 #pragma unroll
@@ -465,31 +506,42 @@ __global__ __launch_bounds__(256) void latent_attn_combine_kernel(LatAttnArgs p,
         const float mi = p.ws[(blk0 + i) * stride + row];
         if (mi != -__builtin_huge_valf()) l += p.ws[(blk0 + i) * stride + MQ + row] * exp2f(mi - m);
     }
-    bf16_t* orow = (bf16_t*)p.O + ((int64_t)p.q_row0[s] + tok) * p.ldo + (int64_t)head * p.o_hs;
+    const int64_t o0 = ((int64_t)p.q_row0[s] + tok) * p.ldo + (int64_t)head * p.o_hs;
     for (int dv = lane; dv < p.DV; dv += 64) {
         float acc = 0.f;
         for (int i = 0; i < p.splits; ++i) {
-            const float mi = p.ws[(blk0 + i) * stride + row];
-            if (mi != -__builtin_huge_valf()) acc += p.ws[(blk0 + i) * stride + 2 * MQ + (int64_t)row * DVP + dv] * exp2f(mi - m);
+            const float mi = p.ws[(blk0 + i) * stride + row], w = p.ws[(blk0 + i) * stride + 2 * MQ + (int64_t)row * DVP + dv];
+            if (p.sig_bias) acc += w;  // sigmoid weights simply add up
+            else if (mi != -__builtin_huge_valf()) acc += w * exp2f(mi - m);
         }
-        orow[dv] = f2bf(acc / l);
+        const float v = p.sig_bias ? acc : acc / l;
+        if (p.o_dt == MI355_DT_F32) ((float*)p.O)[o0 + dv] = v;
+        else ((bf16_t*)p.O)[o0 + dv] = f2bf(v);
     }
 }
 
-template <int DKS>
+template <int DKS, bool SIG>
 static int launch_mfma(const LatAttnArgs& p, dim3 grid, int vec_ok, hipStream_t st) {
-    if (p.DV <= 32) latent_attn_mfma_kernel<DKS, 1><<<grid, 256, 0, st>>>(p, vec_ok);
-    else if (p.DV <= 64) latent_attn_mfma_kernel<DKS, 2><<<grid, 256, 0, st>>>(p, vec_ok);
-    else if (p.DV <= 128) latent_attn_mfma_kernel<DKS, 4><<<grid, 256, 0, st>>>(p, vec_ok);
-    else latent_attn_mfma_kernel<DKS, 8><<<grid, 256, 0, st>>>(p, vec_ok);
+    if (p.DV <= 32) latent_attn_mfma_kernel<DKS, 1, SIG><<<grid, 256, 0, st>>>(p, vec_ok);
+    else if (p.DV <= 64) latent_attn_mfma_kernel<DKS, 2, SIG><<<grid, 256, 0, st>>>(p, vec_ok);
+    else if (p.DV <= 128) latent_attn_mfma_kernel<DKS, 4, SIG><<<grid, 256, 0, st>>>(p, vec_ok);
+    else latent_attn_mfma_kernel<DKS, 8, SIG><<<grid, 256, 0, st>>>(p, vec_ok);
     return 0;
+}
+template <bool SIG>
+static int launch_mfma_dk(const LatAttnArgs& p, dim3 grid, int vec_ok, hipStream_t st) {
+    const int DK = p.D1 + p.D2;
+    if (DK <= 64) return launch_mfma<8, SIG>(p, grid, vec_ok, st);
+    if (DK <= 128) return launch_mfma<16, SIG>(p, grid, vec_ok, st);
+    if (DK <= 192) return launch_mfma<24, SIG>(p, grid, vec_ok, st);
+    return launch_mfma<40, SIG>(p, grid, vec_ok, st);
 }
 
 extern "C" int mi355_latent_attn(int n_seq, int max_new, int H, int hm, int D1, int D2, int DV, const float* Q, int64_t ldq, int q_hs, const void* K1, int64_t ldk1,
                                  int k1_hs, const void* K2, int64_t ldk2, const void* V, int64_t ldv, int v_hs, void* O, int64_t ldo, int o_hs, int dt,
                                  const int* q_row0, const int* n_new, const int* past, const int* k1_row0, const int* k2_row0, const int* v_row0, float scale,
                                  int use_mfma, int splits, float* ws, int64_t ws_floats, int kv_rep, int window, int keep_first, float softcap, const float* sink,
-                                 int pool, const void* PK, const void* PV, int64_t ldp, const int* pool_row0, int chunk, void* stream) {
+                                 int pool, const void* PK, const void* PV, int64_t ldp, const int* pool_row0, int chunk, const float* sig_bias, int o_dt, void* stream) {
     MI355_REQUIRE(n_seq > 0 && n_seq <= 65535 && max_new > 0 && H > 0 && D1 > 0 && D2 >= 0 && DV > 0 && DV <= 512 && Q && K1 && V && O && (D2 == 0 || K2),
                   "latent_attn: bad arguments (value width <= 512)");
     MI355_REQUIRE(dt == MI355_DT_BF16 || dt == MI355_DT_F32, "latent_attn: bad dtype");
@@ -502,6 +554,8 @@ extern "C" int mi355_latent_attn(int n_seq, int max_new, int H, int hm, int D1, 
     MI355_REQUIRE(pool == 0 || (window > 0 && keep_first == 0 && D2 == 0 && PK && PV && pool_row0 && ldp >= (int64_t)((H - 1) / kv_rep) * k1_hs + D1 &&
                                 ldp >= (int64_t)((H - 1) / kv_rep) * v_hs + DV),
                   "latent_attn: pooled blocks need a window, one-part keys and the pooled rows (laid out like the key / value rows)");
+    MI355_REQUIRE(o_dt == MI355_DT_BF16 || o_dt == MI355_DT_F32, "latent_attn: bad output dtype");
+    MI355_REQUIRE(!sig_bias || (softcap == 0.f && !sink), "latent_attn: sigmoid weights combine with neither a cap nor a sink");
     MI355_REQUIRE(q_row0 && n_new && past && k1_row0 && k2_row0 && v_row0, "latent_attn: sequence descriptors missing");
     MI355_REQUIRE(ldq >= (int64_t)(H - 1) * q_hs + D1 + D2 && ldo >= (int64_t)(H - 1) * o_hs + DV && ldk1 >= (int64_t)((H - 1) / kv_rep) * k1_hs + D1 && ldv >= (int64_t)((H - 1) / kv_rep) * v_hs + DV &&
                       (D2 == 0 || ldk2 >= D2),
@@ -516,6 +570,7 @@ extern "C" int mi355_latent_attn(int n_seq, int max_new, int H, int hm, int D1, 
     p.kv_rep = kv_rep, p.window = window, p.keep_first = keep_first, p.chunk = chunk;
     p.softcap = softcap, p.sink = sink, p.pool = pool, p.PK = PK, p.PV = PV, p.ldp = ldp, p.pool_row0 = pool_row0;
     p.splits = 1, p.ws = nullptr;
+    p.sig_bias = sig_bias, p.o_dt = o_dt;
     const bool mfma = use_mfma && D1 + D2 <= 320 && DV <= 256;  // what the MFMA kernel keeps in registers; larger heads take the FMA path
     const int tm = (mfma ? MQ : AM) / hm;
     const int64_t gx = ((int64_t)max_new + tm - 1) / tm, gy = (H + hm - 1) / hm;
@@ -532,11 +587,8 @@ extern "C" int mi355_latent_attn(int n_seq, int max_new, int H, int hm, int D1, 
         const int vec_ok = D1 % 8 == 0 && D2 % 8 == 0 && DV % 8 == 0 && ldk1 % 8 == 0 && ldk2 % 8 == 0 && ldv % 8 == 0 && k1_hs % 8 == 0 && v_hs % 8 == 0 &&
                            ((uintptr_t)K1 & 15) == 0 && ((uintptr_t)K2 & 15) == 0 && ((uintptr_t)V & 15) == 0 &&
                            (pool == 0 || (ldp % 8 == 0 && ((uintptr_t)PK & 15) == 0 && ((uintptr_t)PV & 15) == 0));
-        const int DK = D1 + D2;
-        if (DK <= 64) launch_mfma<8>(p, grid, vec_ok, ST(stream));
-        else if (DK <= 128) launch_mfma<16>(p, grid, vec_ok, ST(stream));
-        else if (DK <= 192) launch_mfma<24>(p, grid, vec_ok, ST(stream));
-        else launch_mfma<40>(p, grid, vec_ok, ST(stream));
+        if (sig_bias) launch_mfma_dk<true>(p, grid, vec_ok, ST(stream));
+        else launch_mfma_dk<false>(p, grid, vec_ok, ST(stream));
         MI355_LAUNCH_CHECK("latent_attn(mfma)");
         if (p.splits > 1) {
             const int DVPh = DV <= 32 ? 32 : DV <= 64 ? 64 : DV <= 128 ? 128 : 256;

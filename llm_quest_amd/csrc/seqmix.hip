@@ -544,7 +544,8 @@ extern "C" int mi355_router_logits(int64_t tokens, int E, int K, const float* x,
 // s = sigmoid(logits); choice = s + correction.  Experts form `groups` equal runs of neighbours; a group's score is the sum of its two largest
 // choice scores; only experts of the `keep` best groups may be chosen; the `top` largest allowed choice scores win (ties: lowest index).
 // weights = s of the winners / (their sum + 1e-20) * scale.  One wave per token, expert e on lane e % 64, register e / 64.
-// mode 1 (softmax router): s = softmax(logits) over ALL experts, choice = s (no correction, no groups), weights = s of the winners * scale, not renormalised.
+// mode 1 (softmax router): s = softmax(logits) over ALL experts, choice = s (no correction), a group's score is its LARGEST choice score, weights = s of the
+// winners * scale, not renormalised.
 // mode 2 (softmax over the winners): as mode 1 on logits + correction (a bias that counts for choice and weight), the winners' s divided by their sum --
 // the softmax over the chosen logits alone -- times scale.
 template <int EPL>
@@ -589,7 +590,7 @@ __global__ __launch_bounds__(256) void moe_route_kernel(int64_t T, int E, int to
                 }
             }
         }
-        if (mode == 0 && groups > 1) {
+        if (mode <= 1 && groups > 1) {
             const int per = E / groups;
             // group scores: lane g keeps the score of group g (+ 64 * register)
             float gs[EPL];
@@ -615,7 +616,7 @@ __global__ __launch_bounds__(256) void moe_route_kernel(int64_t T, int E, int to
                     if (e < E && e / per == g && e != bi && c[j] > second) second = c[j];
                 }
                 second = wave_max(second);
-                const float score = per > 1 ? best + second : best;
+                const float score = mode == 0 && per > 1 ? best + second : best;
 #pragma unroll
                 for (int j = 0; j < EPL; ++j)
                     if (lane + 64 * j == g) gs[j] = score;

@@ -5,9 +5,10 @@
 //   * token shift: several learned blends of a row with the previous token's row, the last row carried per sequence;
 //   * a linear recurrence over a matrix state per head in two flavours -- read-then-update with a bonus for the current token and a decay per key channel
 //     (time mixing with data-dependent decay), update-then-read with one decay per head and token, a step size on the value and a skip term (state-space duality);
-//   * the real-gated linear recurrent unit: a diagonal recurrence per channel with input and recurrence gates;
+//   * the real-gated linear recurrent unit: a diagonal recurrence per channel with input and recurrence gates; the minimal gated recurrence, whose gate reads the
+//     current token alone, on the same tiled scan;
 //   * RMS norm in groups of a row with a full-length weight and a SiLU gate before or after it;
-//   * small row-wise activations: squared ReLU, tanh, one sigmoid gate per head.
+//   * small row-wise activations: squared ReLU, tanh, one sigmoid gate per head, a tanh cap.
 //
 // Conventions as in seqmix.hip / seqrec.hip: operands come as bf16 or fp32 (a MI355_DT_* code each); the residual stream, norm statistics, decays, gates
 // of a recurrence and recurrent state are fp32 in both modes.  A "row" is a token of the packed batch; sequences are described by int32 device arrays.
@@ -492,6 +493,73 @@ extern "C" int mi355_rglru_ragged(int n_seq, int C, int blocks, float decay_c, c
     return 0;
 }
 
+// ------------------------------------------------------------------------------------------- minimal gated recurrence
+// Per channel: z = sigmoid(zr), candidate = u + 1/2 (u >= 0) or sigmoid(u) (u < 0); S <- (1 - z) S + z * candidate; out[t, c] = S * silu(g).  The gate reads the
+// current token only, so the step is an affine map of S known ahead of time and the scan is the one of rglru_kernel: a workgroup = 64 channels x RG_W waves,
+// RG_TB tokens per wave from zero, (product, value) pairs through LDS.  1 - z = sigmoid(-zr).
+__device__ __forceinline__ float sigmoid_p(float v) { return 1.0f / (1.0f + expf(-v)); }
+__global__ __launch_bounds__(64 * RG_W) void mingru_kernel(int n_seq, int C, const float* __restrict__ zr, int64_t ldz, const float* __restrict__ x, int64_t ldx,
+                                                           const void* __restrict__ g, int g_dt, int64_t ldg, const int* __restrict__ seq_off, const int* __restrict__ slot,
+                                                           float* __restrict__ state, void* __restrict__ out, int out_dt, int64_t ldo) {
+    __shared__ float sP[RG_W][64], sL[RG_W][64];
+    const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
+    const int ctiles = (C + 63) / 64;
+    const int s = blockIdx.x / ctiles, c = (blockIdx.x % ctiles) * 64 + lane;
+    const bool ok = c < C;
+    const int cc = ok ? c : 0;
+    float S = state[(int64_t)slot[s] * C + cc];  // the state the tile comes in with (every wave keeps its own copy)
+    const int t0 = seq_off[s], t1 = seq_off[s + 1];
+    float nz[RG_TB], nx[RG_TB], ng[RG_TB];
+    auto fetch = [&](int tb) {
+#pragma unroll
+        for (int q = 0; q < RG_TB; ++q) {
+            const int64_t t = min(tb + q, t1 - 1);
+            nz[q] = zr[t * ldz + cc], nx[q] = x[t * ldx + cc], ng[q] = ldp_dt(g, g_dt, t * ldg + cc);
+        }
+    };
+    if (t0 + w * RG_TB < t1) fetch(t0 + w * RG_TB);
+    for (int tile = t0; tile < t1; tile += RG_W * RG_TB) {
+        const int tb = tile + w * RG_TB;  // this wave's first token
+        float P[RG_TB], L[RG_TB], gv[RG_TB];
+        float pa = 1.f, ls = 0.f;
+#pragma unroll
+        for (int q = 0; q < RG_TB; ++q) {
+            if (tb + q < t1) {
+                const float keep = sigmoid_p(-nz[q]), cand = nx[q] >= 0.f ? nx[q] + 0.5f : sigmoid_p(nx[q]);
+                ls = keep * ls + sigmoid_p(nz[q]) * cand;
+                pa *= keep;
+                gv[q] = silu_p(ng[q]);
+            }
+            P[q] = pa, L[q] = ls;
+        }
+        if (tb + RG_W * RG_TB < t1) fetch(tb + RG_W * RG_TB);
+        sP[w][lane] = pa, sL[w][lane] = ls;  // a wave whose tokens lie past the sequence's end leaves (1, 0): the identity
+        __syncthreads();
+        float sin = S, send = S;
+#pragma unroll
+        for (int v = 0; v < RG_W; ++v) {
+            send = sP[v][lane] * send + sL[v][lane];
+            if (v + 1 == w) sin = send;
+        }
+#pragma unroll
+        for (int q = 0; q < RG_TB; ++q)
+            if (ok && tb + q < t1) stp_dt(out, out_dt, (int64_t)(tb + q) * ldo + c, (L[q] + P[q] * sin) * gv[q]);
+        S = send;
+        __syncthreads();
+    }
+    if (ok && w == 0) state[(int64_t)slot[s] * C + c] = S;
+}
+
+extern "C" int mi355_mingru_ragged(int n_seq, int C, const float* zr, int64_t ldz, const float* x, int64_t ldx, const void* g, int g_dt, int64_t ldg, const int* seq_off,
+                                   const int* slot, float* state, void* out, int out_dt, int64_t ldo, void* stream) {
+    MI355_REQUIRE(n_seq > 0 && C > 0 && zr && x && g && seq_off && slot && state && out && par_dt_ok(g_dt) && par_dt_ok(out_dt) && ldz >= C && ldx >= C && ldg >= C && ldo >= C &&
+                      (int64_t)n_seq * ((C + 63) / 64) < ((int64_t)1 << 31),
+                  "mingru_ragged: bad arguments");
+    mingru_kernel<<<(unsigned)((int64_t)n_seq * ((C + 63) / 64)), 64 * RG_W, 0, ST(stream)>>>(n_seq, C, zr, ldz, x, ldx, g, g_dt, ldg, seq_off, slot, state, out, out_dt, ldo);
+    MI355_LAUNCH_CHECK("mingru_ragged");
+    return 0;
+}
+
 // ------------------------------------------------------------------------------------------- RMS norm in groups with a SiLU gate
 // o fp32 [T, n] cut into `groups` equal consecutive groups; w fp32 [n].  gate_first 0: out = o / rms_group(o) * w * silu(gate);
 // gate_first 1: g = o * silu(gate), out = g / rms_group(g) * w.  One wave per (row, group).
@@ -527,9 +595,9 @@ extern "C" int mi355_gated_groupnorm(int64_t tokens, int n, int groups, const fl
 }
 
 // ------------------------------------------------------------------------------------------- small row-wise activations
-// kind 0: relu(x)^2.  kind 1: tanh(x).  kind 2: x[r, i] * sigmoid(gate[r, i / group]) -- one gate per run of `group` entries (a head).
+// kind 0: relu(x)^2.  kind 1: tanh(x).  kind 2: x[r, i] * sigmoid(gate[r, i / group]) -- one gate per run of `group` entries (a head).  kind 3: limit * tanh(x / limit).
 __global__ __launch_bounds__(256) void unary_rows_kernel(int64_t R, int n, const void* __restrict__ x, int x_dt, int64_t ldx, int kind, const void* __restrict__ gate, int g_dt,
-                                                         int64_t ldg, int group, void* __restrict__ out, int out_dt, int64_t ldo) {
+                                                         int64_t ldg, int group, float limit, void* __restrict__ out, int out_dt, int64_t ldo) {
     const int64_t total = R * n;
     for (int64_t e = (int64_t)blockIdx.x * blockDim.x + threadIdx.x; e < total; e += (int64_t)gridDim.x * blockDim.x) {
         const int64_t r = e / n;
@@ -538,13 +606,14 @@ __global__ __launch_bounds__(256) void unary_rows_kernel(int64_t R, int n, const
         float v;
         if (kind == 0) v = a > 0.f ? a * a : 0.f;
         else if (kind == 1) v = tanhf(a);
+        else if (kind == 3) v = limit * tanhf(a / limit);
         else v = a / (1.0f + expf(-ldp_dt(gate, g_dt, r * ldg + i / group)));
         stp_dt(out, out_dt, r * ldo + i, v);
     }
 }
 template <int KIND>
 __global__ __launch_bounds__(256) void unary_rows_vec_kernel(int64_t R, int n, const void* __restrict__ x, int x_dt, int64_t ldx, const void* __restrict__ gate, int g_dt,
-                                                             int64_t ldg, int group, void* __restrict__ out, int out_dt, int64_t ldo) {
+                                                             int64_t ldg, int group, float limit, void* __restrict__ out, int out_dt, int64_t ldo) {
     const int n4 = n / 4;
     const int64_t total = R * n4;
     for (int64_t e = (int64_t)blockIdx.x * blockDim.x + threadIdx.x; e < total; e += (int64_t)gridDim.x * blockDim.x) {
@@ -556,25 +625,27 @@ __global__ __launch_bounds__(256) void unary_rows_vec_kernel(int64_t R, int n, c
             a = a * sg;
         } else {
 #pragma unroll
-            for (int q = 0; q < 4; ++q) a[q] = KIND == 0 ? (a[q] > 0.f ? a[q] * a[q] : 0.f) : tanhf(a[q]);
+            for (int q = 0; q < 4; ++q) a[q] = KIND == 0 ? (a[q] > 0.f ? a[q] * a[q] : 0.f) : KIND == 3 ? limit * tanhf(a[q] / limit) : tanhf(a[q]);
         }
         stp4_dt(out, out_dt, r * ldo + i, a);
     }
 }
 
-extern "C" int mi355_unary_rows(int64_t rows, int n, const void* x, int x_dt, int64_t ldx, int kind, const void* gate, int g_dt, int64_t ldg, int group, void* out,
-                                int out_dt, int64_t ldo, void* stream) {
-    MI355_REQUIRE(rows > 0 && n > 0 && x && out && par_dt_ok(x_dt) && par_dt_ok(out_dt) && ldx >= n && ldo >= n && kind >= 0 && kind <= 2, "unary_rows: bad arguments");
+extern "C" int mi355_unary_rows(int64_t rows, int n, const void* x, int x_dt, int64_t ldx, int kind, const void* gate, int g_dt, int64_t ldg, int group, float limit,
+                                void* out, int out_dt, int64_t ldo, void* stream) {
+    MI355_REQUIRE(rows > 0 && n > 0 && x && out && par_dt_ok(x_dt) && par_dt_ok(out_dt) && ldx >= n && ldo >= n && kind >= 0 && kind <= 3 && (kind != 3 || limit > 0.f),
+                  "unary_rows: bad arguments");
     MI355_REQUIRE(kind != 2 || (gate && par_dt_ok(g_dt) && group >= 1 && ldg >= (n + group - 1) / group), "unary_rows: a head gate needs its rows and the head size");
-    if ((kind < 2 || group % 4 == 0) && n % 4 == 0 && ldx % 4 == 0 && ldo % 4 == 0 && par_al16(x) && par_al16(out)) {
+    if ((kind != 2 || group % 4 == 0) && n % 4 == 0 && ldx % 4 == 0 && ldo % 4 == 0 && par_al16(x) && par_al16(out)) {
         const int g4 = par_grid(rows * (n / 4), 256, 65535 * 8);
-        if (kind == 0) unary_rows_vec_kernel<0><<<g4, 256, 0, ST(stream)>>>(rows, n, x, x_dt, ldx, gate, g_dt, ldg, group, out, out_dt, ldo);
-        else if (kind == 1) unary_rows_vec_kernel<1><<<g4, 256, 0, ST(stream)>>>(rows, n, x, x_dt, ldx, gate, g_dt, ldg, group, out, out_dt, ldo);
-        else unary_rows_vec_kernel<2><<<g4, 256, 0, ST(stream)>>>(rows, n, x, x_dt, ldx, gate, g_dt, ldg, group, out, out_dt, ldo);
+        if (kind == 0) unary_rows_vec_kernel<0><<<g4, 256, 0, ST(stream)>>>(rows, n, x, x_dt, ldx, gate, g_dt, ldg, group, limit, out, out_dt, ldo);
+        else if (kind == 1) unary_rows_vec_kernel<1><<<g4, 256, 0, ST(stream)>>>(rows, n, x, x_dt, ldx, gate, g_dt, ldg, group, limit, out, out_dt, ldo);
+        else if (kind == 3) unary_rows_vec_kernel<3><<<g4, 256, 0, ST(stream)>>>(rows, n, x, x_dt, ldx, gate, g_dt, ldg, group, limit, out, out_dt, ldo);
+        else unary_rows_vec_kernel<2><<<g4, 256, 0, ST(stream)>>>(rows, n, x, x_dt, ldx, gate, g_dt, ldg, group, limit, out, out_dt, ldo);
         MI355_LAUNCH_CHECK("unary_rows");
         return 0;
     }
-    unary_rows_kernel<<<par_grid(rows * n, 256, 65535 * 8), 256, 0, ST(stream)>>>(rows, n, x, x_dt, ldx, kind, gate, g_dt, ldg, group, out, out_dt, ldo);
+    unary_rows_kernel<<<par_grid(rows * n, 256, 65535 * 8), 256, 0, ST(stream)>>>(rows, n, x, x_dt, ldx, kind, gate, g_dt, ldg, group, limit, out, out_dt, ldo);
     MI355_LAUNCH_CHECK("unary_rows");
     return 0;
 }

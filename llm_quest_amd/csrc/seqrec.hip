@@ -353,13 +353,13 @@ struct QkvRowsArgs {
     float* q_out;
     void* cache;
     int64_t lds_, ldq, ldc;
-    int src_dt, c_dt, H, G, d, dv, dims, layout;
+    int src_dt, c_dt, H, G, GV, d, dv, dims, layout;  // H query heads and G key heads of d, GV value heads of dv
     float eps;
 };
 
 __global__ __launch_bounds__(256) void qkv_rows_kernel(int64_t T, QkvRowsArgs p) {
     const int lane = threadIdx.x & 63;
-    const int HT = p.H + 2 * p.G;
+    const int HT = p.H + p.G + p.GV;
     const int64_t items = T * HT;
     for (int64_t it = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6); it < items; it += (int64_t)gridDim.x * 4) {
         const int64_t t = it / HT;
@@ -413,16 +413,17 @@ __global__ __launch_bounds__(256) void qkv_rows_kernel(int64_t T, QkvRowsArgs p)
 extern "C" int mi355_qkv_rows_append(int64_t tokens, int H, int G, int d, int dv, const void* src, int src_dt, int64_t ld_src, const float* bias, const float* qw,
                                      const float* kw, float eps, const float* qscale, int dims, int layout, const float* freq, const int* pos, const int* dst_row,
                                      float* q_out, int64_t ldq, void* cache, int c_dt, int64_t ldc, float qt_coef, int qt_every, const float* vmix, int64_t ldvm,
-                                     float lam, void* stream) {
-    MI355_REQUIRE(qt_every >= 0 && (!vmix || ldvm >= (int64_t)G * dv), "qkv_rows_append: bad query temperature or value-mix rows");
+                                     float lam, int v_heads, void* stream) {
+    const int GV = v_heads > 0 ? v_heads : G;
+    MI355_REQUIRE(qt_every >= 0 && v_heads >= 0 && (!vmix || ldvm >= (int64_t)GV * dv), "qkv_rows_append: bad query temperature, value heads or value-mix rows");
     MI355_REQUIRE(tokens > 0 && H > 0 && G > 0 && d > 0 && dv > 0 && src && pos && dst_row && q_out && cache && rec_dt_ok(src_dt) && rec_dt_ok(c_dt), "qkv_rows_append: bad arguments");
     MI355_REQUIRE(dims >= 0 && dims % 2 == 0 && dims <= d && (dims == 0 || freq) && (layout == 0 || layout == 1), "qkv_rows_append: the rotated range must lie inside a head");
-    MI355_REQUIRE(ld_src >= (int64_t)(H + G) * d + (int64_t)G * dv && ldq >= (int64_t)H * d && ldc >= (int64_t)G * (d + dv), "qkv_rows_append: rows too short");
+    MI355_REQUIRE(ld_src >= (int64_t)(H + G) * d + (int64_t)GV * dv && ldq >= (int64_t)H * d && ldc >= (int64_t)G * d + (int64_t)GV * dv, "qkv_rows_append: rows too short");
     QkvRowsArgs p;
     p.src = src, p.bias = bias, p.qw = qw, p.kw = kw, p.qscale = qscale, p.freq = freq, p.pos = pos, p.dst_row = dst_row, p.q_out = q_out, p.cache = cache;
-    p.lds_ = ld_src, p.ldq = ldq, p.ldc = ldc, p.src_dt = src_dt, p.c_dt = c_dt, p.H = H, p.G = G, p.d = d, p.dv = dv, p.dims = dims, p.layout = layout, p.eps = eps;
+    p.lds_ = ld_src, p.ldq = ldq, p.ldc = ldc, p.src_dt = src_dt, p.c_dt = c_dt, p.H = H, p.G = G, p.GV = GV, p.d = d, p.dv = dv, p.dims = dims, p.layout = layout, p.eps = eps;
     p.vmix = vmix, p.ldvm = ldvm, p.lam = lam, p.qt_coef = qt_coef, p.qt_every = qt_every;
-    qkv_rows_kernel<<<rec_rows_grid(tokens * (H + 2 * G), 4), 256, 0, ST(stream)>>>(tokens, p);
+    qkv_rows_kernel<<<rec_rows_grid(tokens * (H + G + GV), 4), 256, 0, ST(stream)>>>(tokens, p);
     MI355_LAUNCH_CHECK("qkv_rows_append");
     return 0;
 }

@@ -2,7 +2,8 @@
 post-sum LayerNorm on an fp32 residual stream, latent key/value rows, rotary embedding in both pair layouts, two-part-key / grouped-query / windowed attention,
 gated linear attention and retention with carried state, the sigmoid and softmax routers and the grouped expert products (with gated epilogues), the residual
 sum with RMS norms in groups, short convolutions with carried inputs, query / key / value rows into a slot cache, the gated delta rule, gated activations,
-the residual sum between two norms (sandwich norms), pooled key / value rows, xIELU and sigmoid output gates on rows.
+the residual sum between two norms (sandwich norms), pooled key / value rows, xIELU and sigmoid output gates on rows, the sum of parallel sublayers with a depth
+average, the join of differential attention (csrc/seqpar.hip, csrc/seqdep.hip).
 
 Activations are bf16 (serving mode: bf16 operands, fp32 accumulation) or fp32 (true 32-bit mode: every product is an fp32 FMA chain; the bf16
 weights are exactly representable and widened on load).  Whatever the mode, the residual stream, norm statistics, rotary angles, decays,
@@ -31,8 +32,8 @@ def _i32(t, name, n=None):
         raise ValueError(f"{name}: contiguous int32 tensor{'' if n is None else f' of at least {n} entries'} required")
 
 
-def embed_hash(tok, prev, table, scale, bigram=None, buckets=0, mul_prev=0, mul_cur=0):
-    """fp32 [tokens, width] = table[tok] * scale (+ bigram row hashed from (prev, tok); prev < 0 selects row ``buckets``)."""
+def embed_hash(tok, prev, table, scale, bigram=None, buckets=0, mul_prev=0, mul_cur=0, out=None):
+    """fp32 [tokens, width] = table[tok] * scale (+ bigram row hashed from (prev, tok); prev < 0 selects row ``buckets``); into ``out`` if given."""
     L.require_gpu(tok, prev, table, bigram)
     T = tok.numel()
     _i32(tok, "embed_hash(tok)")
@@ -42,7 +43,10 @@ def embed_hash(tok, prev, table, scale, bigram=None, buckets=0, mul_prev=0, mul_
             raise ValueError("embed_hash: the bigram table is bf16 [buckets + 1, width]")
     if table.dtype != BF16 or not table.is_contiguous():
         raise ValueError("embed_hash: the table is contiguous bf16")
-    out = torch.empty((T, table.shape[1]), dtype=F32, device=table.device)
+    if out is None:
+        out = torch.empty((T, table.shape[1]), dtype=F32, device=table.device)
+    elif out.dtype != F32 or not out.is_contiguous() or tuple(out.shape) != (T, table.shape[1]):
+        raise ValueError("embed_hash: out is contiguous fp32 [tokens, width]")
     L.call("mi355_embed_hash_fwd", T, table.shape[1], table.shape[0], L.ptr(tok), L.ptr(prev), L.ptr(table), float(scale), L.ptr(bigram), int(buckets),
            int(mul_prev), int(mul_cur), L.ptr(out))
     return out
@@ -176,7 +180,7 @@ def router_logits(x32, w):
 
 def moe_route(logits, correction, top, groups, keep, scale, softmax=False):
     """(ids int32 [tokens, top], weights fp32 [tokens, top]).  ``softmax`` True: scores are the softmax over all experts, the winners' scores times ``scale``
-    are the weights (not renormalised); ``softmax`` "chosen": ``correction`` is a bias on the logits, the ``top`` largest win and their weights are the
+    are the weights (not renormalised; of several groups the ``keep`` with the largest members stay eligible); ``softmax`` "chosen": ``correction`` is a bias on the logits, the ``top`` largest win and their weights are the
     softmax over the winners' logits alone (times ``scale``); otherwise the grouped sigmoid router."""
     L.require_gpu(logits, correction)
     if logits.dtype != F32 or not logits.is_contiguous() or (correction is not None and (correction.dtype != F32 or correction.numel() != logits.shape[1])):
@@ -247,15 +251,16 @@ def attn_key_splits(n_seq, head_tiles, max_new, hm, max_keys, per_split=256):
 
 
 def latent_attn(q, k1, k2, v, out, H, hm, D1, D2, DV, q_hs, k1_hs, v_hs, o_hs, desc, max_new, scale, max_keys=0, kv_rep=1, window=0, keep_first=0, softcap=0.0,
-                sink=None, pool=0, pooled=None, pool_row0=None, chunk=0):
+                sink=None, pool=0, pooled=None, pool_row0=None, chunk=0, sig_bias=None):
     """Two-part-key causal attention over a ragged batch.  ``desc`` = (q_row0, n_new, past, k1_row0, k2_row0, v_row0) int32 [n_seq] each.  ``max_keys``
     (the longest sequence's keys, if the caller knows it) lets one-token steps over long caches spread a tile's keys over several workgroups.
     ``kv_rep``: query heads per key / value head (strides per key / value head).  ``window`` > 0: a query sees a key only ``window`` positions back, or
     among the first ``keep_first`` of the sequence.  ``softcap`` > 0: scores pass cap * tanh(score / cap).  ``sink`` (fp32 [H]): exp(sink[h]) joins head h's
     denominator.  ``pool`` > 0: ``pooled`` = (pooled keys, pooled values), views laid out like ``k1`` / ``v`` with one mean row per ``pool`` tokens, first row
     of every sequence in ``pool_row0`` (int32 [n_seq]); a query sees the blocks that lie wholly before its window.  ``chunk`` > 0: positions are cut into chunks
-    of that many from the sequence's first token on, and a query sees only the keys of its own chunk."""
-    L.require_gpu(q, k1, k2, v, out, sink, pool_row0, *desc)
+    of that many from the sequence's first token on, and a query sees only the keys of its own chunk.  ``sig_bias`` (fp32 [H]): no softmax, a visible key's weight is
+    sigmoid(score + sig_bias[h]).  ``out`` has the dtype of the values, or fp32."""
+    L.require_gpu(q, k1, k2, v, out, sink, pool_row0, sig_bias, *desc)
     pk = pv = None
     if pool:
         pk, pv = pooled
@@ -267,10 +272,11 @@ def latent_attn(q, k1, k2, v, out, H, hm, D1, D2, DV, q_hs, k1_hs, v_hs, o_hs, d
             raise ValueError("latent_attn: pooled rows share the dtype of keys / values and one row pitch")
     if sink is not None and (sink.dtype != F32 or not sink.is_contiguous() or sink.numel() != H):
         raise ValueError("latent_attn: sink fp32 [H]")
+    _vec32(sig_bias, H, "latent_attn(sig_bias)")
     for t, n in ((q, "q"), (k1, "k1"), (v, "v"), (out, "out")):
         _rows(t, f"latent_attn({n})")
-    if q.dtype != F32 or k1.dtype != v.dtype or out.dtype != v.dtype or (k2 is not None and k2.dtype != v.dtype):
-        raise ValueError("latent_attn: q fp32; keys, values and output share one dtype")
+    if q.dtype != F32 or k1.dtype != v.dtype or out.dtype not in (v.dtype, F32) or (k2 is not None and k2.dtype != v.dtype):
+        raise ValueError("latent_attn: q fp32; keys and values share one dtype, the output has it or is fp32")
     n_seq = desc[0].numel()
     for t in desc:
         _i32(t, "latent_attn(desc)", n_seq)
@@ -296,7 +302,7 @@ def latent_attn(q, k1, k2, v, out, H, hm, D1, D2, DV, q_hs, k1_hs, v_hs, o_hs, d
     L.call("mi355_latent_attn", n_seq, max_new, H, hm, D1, D2, DV, L.ptr(q), q.stride(0), q_hs, L.ptr(k1), k1.stride(0), k1_hs, L.ptr(k2), 0 if k2 is None else k2.stride(0),
            L.ptr(v), v.stride(0), v_hs, L.ptr(out), out.stride(0), o_hs, _dt(v), *[L.ptr(t) for t in desc], float(scale), 1 if mfma else 0, splits, L.ptr(ws),
            0 if ws is None else ws.numel(), int(kv_rep), int(window), int(keep_first), float(softcap or 0.0), L.ptr(sink), int(pool), L.ptr(pk), L.ptr(pv),
-           0 if pk is None else pk.stride(0), L.ptr(pool_row0), int(chunk))
+           0 if pk is None else pk.stride(0), L.ptr(pool_row0), int(chunk), L.ptr(sig_bias), _dt(out))
     return out
 
 
@@ -357,24 +363,25 @@ def ragged_conv(x, w, state, row_seq, seq_off, slot, act=False, residual=False, 
     return y
 
 
-def qkv_rows_append(src, H, G, d, dv, bias, qw, kw, eps, qscale, dims, layout, freq, pos, dst_row, cache2d, q_temp=None, vmix=None, lam=0.0):
+def qkv_rows_append(src, H, G, d, dv, bias, qw, kw, eps, qscale, dims, layout, freq, pos, dst_row, cache2d, q_temp=None, vmix=None, lam=0.0, v_heads=None):
     """Rows [H x d | G x d | G x dv] -> fp32 queries [tokens, H * d] (bias, head norm, rotation, per-head scale) and key / value rows of ``cache2d``.
     ``q_temp`` = (coef, every): the query at position p is also multiplied by 1 + coef * ln(floor((p + 1) / every) + 1).  ``vmix`` (fp32 [tokens, G * dv],
-    any row pitch): the cached value is (1 - lam) v + lam * vmix."""
+    any row pitch): the cached value is (1 - lam) v + lam * vmix.  ``v_heads``: that many value heads instead of G."""
     L.require_gpu(src, bias, qw, kw, qscale, freq, pos, dst_row, cache2d, vmix)
+    GV = v_heads or G
     if vmix is not None:
         _rows(vmix, "qkv_rows_append(vmix)")
-        if vmix.dtype != F32 or tuple(vmix.shape) != (src.shape[0], G * dv):
-            raise ValueError(f"qkv_rows_append: the rows to mix in are fp32 [{src.shape[0]}, {G * dv}]")
+        if vmix.dtype != F32 or tuple(vmix.shape) != (src.shape[0], GV * dv):
+            raise ValueError(f"qkv_rows_append: the rows to mix in are fp32 [{src.shape[0]}, {GV * dv}]")
     coef, every = (float(q_temp[0]), int(q_temp[1])) if q_temp else (0.0, 0)
     if q_temp and every < 1:
         raise ValueError("qkv_rows_append: the query temperature's step is a positive number of positions")
     _rows(src, "qkv_rows_append(src)")
     _rows(cache2d, "qkv_rows_append(cache)")
     T = src.shape[0]
-    if src.shape[1] != (H + G) * d + G * dv or cache2d.shape[1] != G * (d + dv):
+    if src.shape[1] != (H + G) * d + GV * dv or cache2d.shape[1] != G * d + GV * dv:
         raise ValueError("qkv_rows_append: row widths do not match the head layout")
-    for t, n in ((bias, (H + G) * d + G * dv), (qw, d), (kw, d), (qscale, H), (freq, dims // 2)):
+    for t, n in ((bias, (H + G) * d + GV * dv), (qw, d), (kw, d), (qscale, H), (freq, dims // 2)):
         if t is not None and (t.dtype != F32 or not t.is_contiguous() or t.numel() < n):
             raise ValueError("qkv_rows_append: vectors are contiguous fp32 of the layout's sizes")
     _i32(pos, "qkv_rows_append(pos)", T)
@@ -382,7 +389,7 @@ def qkv_rows_append(src, H, G, d, dv, bias, qw, kw, eps, qscale, dims, layout, f
     q = torch.empty((T, H * d), dtype=F32, device=src.device)
     L.call("mi355_qkv_rows_append", T, H, G, d, dv, L.ptr(src), _dt(src), src.stride(0), L.ptr(bias), L.ptr(qw), L.ptr(kw), float(eps), L.ptr(qscale), int(dims), int(layout),
            L.ptr(freq), L.ptr(pos), L.ptr(dst_row), L.ptr(q), q.stride(0), L.ptr(cache2d), _dt(cache2d), cache2d.stride(0), coef, every, L.ptr(vmix),
-           0 if vmix is None else vmix.stride(0), float(lam))
+           0 if vmix is None else vmix.stride(0), float(lam), int(GV))
     return q
 
 
@@ -620,6 +627,26 @@ def rglru(u, gates, gbias, lam, y, blocks, seq_off, slot, state, out_dtype, deca
     return out
 
 
+def mingru(zr, x, g, seq_off, slot, state, out_dtype):
+    """Minimal gated recurrence over a ragged batch: z = sigmoid(zr), candidate x + 1/2 (x >= 0) or sigmoid(x) (x < 0), S <- (1 - z) S + z * candidate.  zr, x
+    fp32 [tokens, C] (biases already added), g [tokens, C]; ``state`` fp32 [slots, C].  Returns S * silu(g)."""
+    L.require_gpu(zr, x, g, seq_off, slot, state)
+    T, C = zr.shape
+    for t, n in ((zr, "zr"), (x, "x"), (g, "g")):
+        _rows(t, f"mingru({n})")
+        if tuple(t.shape) != (T, C) or (n != "g" and t.dtype != F32):
+            raise ValueError("mingru: zr, x fp32 [tokens, C], g [tokens, C]")
+    n_seq = slot.numel()
+    _i32(seq_off, "mingru(seq_off)", n_seq + 1)
+    _i32(slot, "mingru(slot)")
+    if state.dtype != F32 or not state.is_contiguous() or tuple(state.shape[1:]) != (C,):
+        raise ValueError("mingru: state contiguous fp32 [slots, C]")
+    out = torch.empty((T, C), dtype=out_dtype, device=zr.device)
+    L.call("mi355_mingru_ragged", n_seq, C, L.ptr(zr), zr.stride(0), L.ptr(x), x.stride(0), L.ptr(g), _dt(g), g.stride(0), L.ptr(seq_off), L.ptr(slot), L.ptr(state), L.ptr(out),
+           _dt(out), out.stride(0))
+    return out
+
+
 def gated_groupnorm(o, w, gate, groups, eps, out_dtype, gate_first=False):
     """o fp32 [tokens, n] in ``groups`` equal consecutive groups, w fp32 [n]: o / rms_group(o) * w * silu(gate), or -- ``gate_first`` -- the RMS norm of
     o * silu(gate) times w."""
@@ -636,11 +663,12 @@ def gated_groupnorm(o, w, gate, groups, eps, out_dtype, gate_first=False):
     return out
 
 
-UNARY_RELU2, UNARY_TANH, UNARY_HEAD_GATE = 0, 1, 2
+UNARY_RELU2, UNARY_TANH, UNARY_HEAD_GATE, UNARY_SOFTCAP = 0, 1, 2, 3
 
 
-def unary_rows(x, kind, gate=None, group=1, out_dtype=None):
-    """``UNARY_RELU2``: relu(x)^2; ``UNARY_TANH``; ``UNARY_HEAD_GATE``: x[r, i] * sigmoid(gate[r, i // group]) (gate [rows, n / group])."""
+def unary_rows(x, kind, gate=None, group=1, out_dtype=None, limit=0.0):
+    """``UNARY_RELU2``: relu(x)^2; ``UNARY_TANH``; ``UNARY_HEAD_GATE``: x[r, i] * sigmoid(gate[r, i // group]) (gate [rows, n / group]);
+    ``UNARY_SOFTCAP``: limit * tanh(x / limit)."""
     L.require_gpu(x, gate)
     _rows(x, "unary_rows(x)")
     if kind == UNARY_HEAD_GATE:
@@ -649,7 +677,60 @@ def unary_rows(x, kind, gate=None, group=1, out_dtype=None):
             raise ValueError("unary_rows: one gate per run of `group` entries")
     out = torch.empty(x.shape, dtype=out_dtype or x.dtype, device=x.device)
     L.call("mi355_unary_rows", x.shape[0], x.shape[1], L.ptr(x), _dt(x), x.stride(0), int(kind), L.ptr(gate), 0 if gate is None else _dt(gate),
-           0 if gate is None else gate.stride(0), int(group), L.ptr(out), _dt(out), out.stride(0))
+           0 if gate is None else gate.stride(0), int(group), float(limit), L.ptr(out), _dt(out), out.stride(0))
+    return out
+
+
+def depth_sum(x, ya=None, ca=1.0, yb=None, cb=1.0, ls1=None, y2=None, parts=1, ls2=None, hist=None, n_hist=0, d=None, x_out=None, norm=None, eps=0.0, out_dtype=None,
+              want32=False):
+    """The end of a block with parallel sublayers and the start of the next: v = x + ls1 * (ca ya + cb yb) + ls2 * (sum of y2's ``parts`` rows per token); with
+    depth weights ``d`` (fp32 [n_hist + 1]) v becomes result ``n_hist`` of ``hist`` (fp32 [layers + 1, tokens, width]) and the stream goes on as
+    sum_j d[j] hist[j] (j <= n_hist).  ``x_out`` (True: a new tensor, or a tensor, or None) receives it; ``norm`` (fp32 [width]): its RMS norm times that weight
+    is returned in ``out_dtype`` (and as fp32 with ``want32``).  Returns (x_out or None, normed or None, normed fp32 or None)."""
+    L.require_gpu(x, ya, yb, y2, ls1, ls2, hist, d, norm)
+    _rows(x, "depth_sum(x)")
+    T, width = x.shape
+    if x.dtype != F32 or not x.is_contiguous():
+        raise ValueError("depth_sum: x contiguous fp32 [tokens, width]")
+    for y, n, rows in ((ya, "ya", T), (yb, "yb", T), (y2, "y2", T * parts)):
+        if y is not None:
+            _rows(y, f"depth_sum({n})")
+            if tuple(y.shape) != (rows, width):
+                raise ValueError(f"depth_sum({n}): [{rows}, {width}] required, got {tuple(y.shape)}")
+    for v, n in ((ls1, "ls1"), (ls2, "ls2"), (norm, "norm")):
+        _vec32(v, width, f"depth_sum({n})")
+    _vec32(d, n_hist + 1, "depth_sum(d)")
+    if d is not None and (hist is None or hist.dtype != F32 or not hist.is_contiguous() or tuple(hist.shape[1:]) != (T, width) or hist.shape[0] <= n_hist):
+        raise ValueError("depth_sum: the earlier results are contiguous fp32 [> n_hist, tokens, width]")
+    if x_out is True:
+        x_out = torch.empty_like(x)
+    out = out32 = None
+    if norm is not None:
+        od = out_dtype or F32
+        out = torch.empty((T, width), dtype=od, device=x.device)
+        out32 = out if od == F32 else (torch.empty((T, width), dtype=F32, device=x.device) if want32 else None)
+    L.call("mi355_depth_sum", T, width, L.ptr(x), L.ptr(ya), 0 if ya is None else _dt(ya), 0 if ya is None else ya.stride(0), float(ca), L.ptr(yb), 0 if yb is None else _dt(yb),
+           0 if yb is None else yb.stride(0), float(cb), L.ptr(ls1), L.ptr(y2), 0 if y2 is None else _dt(y2), 0 if y2 is None else y2.stride(0), int(parts), L.ptr(ls2),
+           L.ptr(hist), 0 if hist is None else hist.stride(0), int(n_hist), L.ptr(d), L.ptr(x_out), L.ptr(norm), float(eps), L.ptr(out), 0 if out is None else _dt(out),
+           None if out32 is out else L.ptr(out32))
+    return x_out, out, out32
+
+
+def diff_join(a1, a2, H, D, lam, eps, scale, gate, out_dtype):
+    """Differential attention's join: per head o = a1 - lam * a2, divided by its root mean square, times ``scale``, times sigmoid(gate) element by element
+    (``gate`` [tokens, H * D] or None).  a1, a2 fp32 [tokens, H * D]."""
+    L.require_gpu(a1, a2, gate)
+    for t, n in ((a1, "a1"), (a2, "a2")):
+        _rows(t, f"diff_join({n})")
+        if t.dtype != F32 or t.shape[1] != H * D or t.shape[0] != a1.shape[0]:
+            raise ValueError(f"diff_join({n}): fp32 [tokens, {H * D}] required")
+    if gate is not None:
+        _rows(gate, "diff_join(gate)")
+        if gate.shape != a1.shape:
+            raise ValueError("diff_join: the gate has the maps' shape")
+    out = torch.empty(a1.shape, dtype=out_dtype, device=a1.device)
+    L.call("mi355_diff_join", a1.shape[0], H, D, L.ptr(a1), a1.stride(0), L.ptr(a2), a2.stride(0), float(lam), float(eps), float(scale), L.ptr(gate),
+           0 if gate is None else _dt(gate), 0 if gate is None else gate.stride(0), L.ptr(out), _dt(out), out.stride(0))
     return out
 
 

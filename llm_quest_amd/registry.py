@@ -46,10 +46,17 @@ def _gepilix(model_dir, act_dtype, device):
     return load_gepilix(model_dir, act_dtype, device)
 
 
+def _foderax(model_dir, act_dtype, device):
+    from llm_quest_amd.foderax.foderax_weight_loading import load_foderax
+
+    return load_foderax(model_dir, act_dtype, device)
+
+
 register("Gemepel", _gemepel)
 register("Mepatar", _mepatar)
 register("Mopalorn", _mopalorn)
 register("Gepilix", _gepilix)
+register("Foderax", _foderax)
 
 
 def load_model(model_dir, dtype="bfloat16", device="cuda"):
