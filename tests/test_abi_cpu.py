@@ -105,7 +105,7 @@ def test_attention_backward_owned_agprs_are_untouched_by_the_compiler(tmp_path):
         pytest.skip("hipcc not available")
     src = os.path.join(ROOT, "llm_quest_amd", "csrc", "attention.hip")
     out = tmp_path / "attention.s"
-    res = subprocess.run([hipcc, "--offload-arch=gfx950", "-O3", "-std=c++17", "-ffp-contract=off", "-fno-slp-vectorize", "-S", "--cuda-device-only",
+    res = subprocess.run([hipcc, "--offload-arch=gfx950", "-O3", "-std=c++17", "-ffp-contract=off", "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops", "-fno-slp-vectorize", "-S", "--cuda-device-only",
                           "-o", str(out), src], capture_output=True, text=True)
     assert res.returncode == 0, res.stderr[-2000:]
     spec = importlib.util.spec_from_file_location("audit_agpr", os.path.join(ROOT, "tools", "audit_agpr.py"))

@@ -5,7 +5,7 @@
 set -e
 R=$(cd "$(dirname "$0")/.." && pwd); C=$R/llm_quest_amd/csrc; tag=$1; stem=$2; extra=$3
 mkdir -p $R/build_variants/obj
-base="-O3 -std=c++17 -fPIC --offload-arch=gfx950 -Wall -Wno-unused-function -Wno-unused-variable -ffp-contract=off"
+base="-O3 -std=c++17 -fPIC --offload-arch=gfx950 -Wall -Wno-unused-function -Wno-unused-variable -ffp-contract=off -Xclang -target-feature -Xclang -packed-fp32-ops"
 case $stem in
   attention) src=attention.hip; flags="-fno-slp-vectorize";;
   gemm_p*) src=gemm.hip; flags="-DGEMM_PART=${stem#gemm_p}";;
