@@ -842,6 +842,18 @@ class Relu2MLP(_Frozen):
 
 
 # ----------------------------------------------------------------------------------------------- mechanisms of decoders with parallel sublayers and a depth average
+def differential_attention(q, cache2d, H, G, d, dv, scale, lam, eps, out_scale, gate, desc, max_new, max_keys, out_dtype):
+    """Two softmax maps per head over the same values, joined.  q fp32 [tokens, H x 2 d], cache rows [G x 2 d | G x dv] (both head by head as [map 1, map 2]);
+    ``desc`` as ``kernels_seq.latent_attn`` takes it.  Returns unit RMS per head of a1 - lam * a2, times ``out_scale``, times sigmoid(gate)."""
+    maps = []
+    for m in (0, 1):  # the maps' outputs stay fp32: their difference is small where the maps agree
+        a = torch.empty((q.shape[0], H * dv), dtype=F32, device=q.device)
+        S.latent_attn(q[:, m * d :], cache2d[:, m * d :], None, cache2d[:, 2 * G * d :], a, H, _largest_pow2_divisor(H // G), d, 0, dv, 2 * d, 2 * d, dv, dv, desc, max_new, scale,
+                      max_keys=max_keys, kv_rep=H // G)
+        maps.append(a)
+    return S.diff_join(maps[0], maps[1], H, dv, lam, eps, out_scale, gate, out_dtype)
+
+
 class DifferentialAttention(_Frozen):
     """Differential attention: per head two softmax maps (queries and keys of ``dim`` each, laid out head by head as [map 1, map 2]) over the same values
     [``vdim``], grouped queries, biases on q / k / v.  o = a1 - lambda a2 with lambda = exp(lq1 . lk1) - exp(lq2 . lk2) + ``diff``, one number for the layer;
@@ -892,13 +904,9 @@ class DifferentialAttention(_Frozen):
         else:
             q = torch.empty((T, n), dtype=F32, device=h.device)
             S.rope_heads(proj[:, :n], 2 * H, d, d, 0, q, d, 0, 0, self.rot_dims, self.freq, st.pos, layout=self.rot_layout)
-        maps = []
-        for m in (0, 1):  # the maps' outputs stay fp32: their difference is small where the maps agree
-            a = torch.empty((T, H * dv), dtype=F32, device=h.device)
-            S.latent_attn(q[:, m * d :], cache2d[:, m * d :], None, cache2d[:, 2 * G * d :], a, H, _largest_pow2_divisor(H // G), d, 0, dv, 2 * d, 2 * d, dv, dv,
-                          (st.q_row0, st.n_new, st.past, st.cache_row0, st.cache_row0, st.cache_row0), st.max_new, self.scale, max_keys=st.max_keys, kv_rep=H // G)
-            maps.append(a)
-        ctx = S.diff_join(maps[0], maps[1], H, dv, self.lam, self.eps, 1.0 - self.diff, proj[:, n:] if self.gate else None, st.act_dtype)
+        desc = (st.q_row0, st.n_new, st.past, st.cache_row0, st.cache_row0, st.cache_row0)
+        ctx = differential_attention(q, cache2d, H, G, d, dv, self.scale, self.lam, self.eps, 1.0 - self.diff, proj[:, n:] if self.gate else None, desc, st.max_new,
+                                     st.max_keys, st.act_dtype)
         return S.linear(ctx, self.w_o, out_dtype=out_dtype)
 
 
