@@ -661,7 +661,7 @@ int mi355_unary_rows(int64_t rows, int n, const void* x, int x_dt, int64_t ldx, 
 int mi355_mingru_ragged(int n_seq, int C, const float* zr, int64_t ldz, const float* x, int64_t ldx, const void* g, int g_dt, int64_t ldg, const int* seq_off,
                         const int* slot, float* state, void* out, int out_dt, int64_t ldo, void* stream);
 
-/* ---- decoders with parallel sublayers and a depth average in ragged batches (csrc/seqdep.hip) ---- */
+/* ---- decoders with parallel sublayers and a depth average in ragged batches (csrc/seqdep.hip, csrc/latent_attn_full.hip) ---- */
 /* The sum, the depth average and the next norm of a block: v = x[t] + ls1 * (ca * ya[t] + cb * yb[t]) + ls2 * sum_{p < parts} y2[t * parts + p] (ya / yb / y2 may
  * be NULL; ls1 / ls2 fp32 [width], NULL: 1); hist (fp32 [>= n_hist + 1, tokens, width], pitch hist_stride between results): result n_hist <- v;
  * xa = sum_{j < n_hist} d[j] hist[j][t] + d[n_hist] v (d fp32 [n_hist + 1]; d NULL: xa = v, hist may then be NULL); x_out (may be NULL or x) <- xa;
@@ -669,6 +669,14 @@ int mi355_mingru_ragged(int n_seq, int C, const float* zr, int64_t ldz, const fl
 int mi355_depth_sum(int64_t tokens, int width, const float* x, const void* ya, int ya_dt, int64_t ldya, float ca, const void* yb, int yb_dt, int64_t ldyb, float cb,
                     const float* ls1, const void* y2, int y2_dt, int64_t ldy2, int parts, const float* ls2, float* hist, int64_t hist_stride, int n_hist,
                     const float* d, float* x_out, const float* w, float eps, void* out, int out_dt, float* out32, void* stream);
+/* Differential attention in one kernel (bf16 keys and values, fp32 queries, bf16 output): per head two softmax maps over every key j <= i and the same values,
+ * then the join of mi355_diff_join with fp32 gate rows (may be NULL).  Q rows [H x 2 D], key rows [H / kv_rep x 2 D] (head by head [map 1, map 2]), value rows
+ * [H / kv_rep x DV], output rows [H x DV]; sequence descriptors as in mi355_latent_attn.  A tile covers 64 / hm tokens x hm heads (hm divides kv_rep and 32);
+ * splits > 1 deals a tile's keys to that many workgroups (ws: n_seq * head tiles * token tiles * splits * 128 * (2 + DV rounded up to 32 / 64 / 128 / 256) floats).
+ * D <= 128, DV <= 256, multiples of 8, rows 16-byte aligned, scale > 0. */
+int mi355_diff_attn(int n_seq, int max_new, int H, int hm, int D, int DV, const float* Q, int64_t ldq, const void* K, int64_t ldk, const void* V, int64_t ldv,
+                    void* O, int64_t ldo, const int* q_row0, const int* n_new, const int* past, const int* k_row0, float scale, int kv_rep, int splits, float* ws,
+                    int64_t ws_floats, float lam, float eps, float c, const float* gate, int64_t ldg, void* stream);
 /* Join of differential attention: per head of D entries o = a1 - lam * a2 (fp32 rows [H x D]), o / sqrt(mean(o^2) + eps) * c, times sigmoid(gate) element by
  * element (gate rows [H x D] of dtype g_dt, may be NULL). */
 int mi355_diff_join(int64_t tokens, int H, int D, const float* a1, int64_t lda1, const float* a2, int64_t lda2, float lam, float eps, float c, const void* gate, int g_dt,

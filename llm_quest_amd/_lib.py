@@ -134,6 +134,7 @@ SIGNATURES = {
     "mi355_mingru_ragged": [_I, _I, _P, _L, _P, _L, _P, _I, _L, _P, _P, _P, _P, _I, _L, _P],
     # decoders with parallel sublayers and a depth average in ragged batches (csrc/seqdep.hip)
     "mi355_depth_sum": [_L, _I, _P, _P, _I, _L, _F, _P, _I, _L, _F, _P, _P, _I, _L, _I, _P, _P, _L, _I, _P, _P, _P, _F, _P, _I, _P, _P],
+    "mi355_diff_attn": [_I, _I, _I, _I, _I, _I, _P, _L, _P, _L, _P, _L, _P, _L, _P, _P, _P, _P, _F, _I, _I, _P, _L, _F, _F, _F, _P, _L, _P],
     "mi355_diff_join": [_L, _I, _I, _P, _L, _P, _L, _F, _F, _F, _P, _I, _L, _P, _I, _L, _P],
     # measurement aid (csrc/probe.hip)
     "mi355_mfma_pipe_probe": [_I, _I, _P, _P],

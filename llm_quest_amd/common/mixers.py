@@ -844,12 +844,17 @@ class Relu2MLP(_Frozen):
 # ----------------------------------------------------------------------------------------------- mechanisms of decoders with parallel sublayers and a depth average
 def differential_attention(q, cache2d, H, G, d, dv, scale, lam, eps, out_scale, gate, desc, max_new, max_keys, out_dtype):
     """Two softmax maps per head over the same values, joined.  q fp32 [tokens, H x 2 d], cache rows [G x 2 d | G x dv] (both head by head as [map 1, map 2]);
-    ``desc`` as ``kernels_seq.latent_attn`` takes it.  Returns unit RMS per head of a1 - lam * a2, times ``out_scale``, times sigmoid(gate)."""
+    ``desc`` as ``kernels_seq.latent_attn`` takes it.  bf16 keys and values of aligned widths: one kernel for both maps and the join; else a launch per map and the
+    join.  Returns unit RMS per head of a1 - lam * a2, times ``out_scale``, times sigmoid(gate)."""
+    rep = H // G
+    aligned = d % 8 == 0 and dv % 8 == 0 and q.data_ptr() % 16 == 0 and (gate is None or (gate.data_ptr() % 16 == 0 and gate.stride(0) % 4 == 0))
+    if cache2d.dtype == BF16 and out_dtype == BF16 and d <= 128 and dv <= 256 and scale > 0 and aligned:
+        return S.diff_attn(q, cache2d, cache2d[:, 2 * G * d :], H, _largest_pow2_divisor(rep), d, dv, scale, lam, eps, out_scale, gate, desc, max_new, max_keys, rep)
     maps = []
     for m in (0, 1):  # the maps' outputs stay fp32: their difference is small where the maps agree
         a = torch.empty((q.shape[0], H * dv), dtype=F32, device=q.device)
-        S.latent_attn(q[:, m * d :], cache2d[:, m * d :], None, cache2d[:, 2 * G * d :], a, H, _largest_pow2_divisor(H // G), d, 0, dv, 2 * d, 2 * d, dv, dv, desc, max_new, scale,
-                      max_keys=max_keys, kv_rep=H // G)
+        S.latent_attn(q[:, m * d :], cache2d[:, m * d :], None, cache2d[:, 2 * G * d :], a, H, _largest_pow2_divisor(rep), d, 0, dv, 2 * d, 2 * d, dv, dv, desc, max_new, scale,
+                      max_keys=max_keys, kv_rep=rep)
         maps.append(a)
     return S.diff_join(maps[0], maps[1], H, dv, lam, eps, out_scale, gate, out_dtype)
 

@@ -14,37 +14,11 @@
 // Scores, softmax statistics and the output accumulators are fp32.  A tile is `tm` tokens x `hm` heads = 32 query rows (hm > 1 only with shared
 // keys and values) against 64 keys at a time.
 //
-// Two compute paths: fp32 FMA through LDS (any operand type: the true-fp32 mode), and bf16 MFMA (v_mfma_f32_32x32x8_bf16_1k) for bf16 keys / values.
-#include "common.h"
+// Three compute paths: fp32 FMA through LDS (any operand type: the true-fp32 mode), bf16 MFMA (v_mfma_f32_32x32x8_bf16_1k) for bf16 keys / values with every
+// option, and -- latent_attn_full.hip -- a leaner bf16 MFMA kernel for the cases that see every key j <= i without a cap.
+#include "latent_attn.h"
 
 #define ST(s) ((hipStream_t)(s))
-
-struct LatAttnArgs {
-    const float* Q;
-    const void* K1;
-    const void* K2;
-    const void* V;
-    void* O;
-    int64_t ldq, ldk1, ldk2, ldv, ldo;
-    int q_hs, k1_hs, v_hs, o_hs;
-    int D1, D2, DV, H, hm, dt;
-    const int *q_row0, *n_new, *past, *k1_row0, *k2_row0, *v_row0;
-    float scale;
-    int splits;  // MFMA path: a tile's keys are dealt to `splits` workgroups; partial (max, sum, output) rows go to ws and latent_attn_combine_kernel joins them
-    float* ws;   // per (sequence, head tile, token tile, split): 128 maxima | 128 sums | 128 x DVP unnormalised outputs
-    int kv_rep;  // query heads per key / value head (grouped queries): head h reads key / value head h / kv_rep
-    int window;  // > 0: a query at position i sees key j <= i only if i - j < window or j < keep_first (sliding window that keeps the first tokens)
-    int keep_first;
-    int chunk;  // > 0: positions are cut into chunks of this many, counted from the sequence's first token; a query sees only the keys of its own chunk
-    float softcap;      // > 0: score <- softcap * tanh(score / softcap) after the scale
-    const float* sink;  // fp32 [H] or NULL: exp(sink[h]) joins the denominator of head h (no key, no value, not scaled)
-    int pool;           // > 0: one pooled key / value row per `pool` tokens (needs window > 0, D2 == 0); rows PK / PV, first row of sequence s = pool_row0[s]
-    const void *PK, *PV;
-    int64_t ldp;
-    const int* pool_row0;
-    const float* sig_bias;  // fp32 [H] or NULL: weights sigmoid(score + sig_bias[head]) instead of a softmax
-    int o_dt;               // dtype of the output rows (MI355_DT_*)
-};
 
 // pooled blocks the query at position lim sees: those that end at or before lim - window
 __device__ __forceinline__ int pooled_visible(int lim, int window, int pool) {
@@ -66,7 +40,7 @@ __device__ __forceinline__ int tile_key_floor(int pos0, int window, int chunk) {
 
 __device__ __forceinline__ float lda_dt(const void* p, int dt, int64_t i) { return dt == MI355_DT_F32 ? ((const float*)p)[i] : bf2f(((const bf16_t*)p)[i]); }
 
-#define AM 32  // query rows per tile
+#define AM 32  // query rows per tile of the FMA kernel
 #define AN 64  // keys per step
 #define AC 32  // feature chunk of the score product
 
@@ -245,7 +219,7 @@ __global__ __launch_bounds__(256) void latent_attn_fma_kernel(LatAttnArgs p) {
 // query), so a lane holds 16 of every 32 keys of ONE query: the softmax statistics are lane-local plus one exchange with lane ^ 32, the rescale factor
 // of the transposed output O^T = V^T P^T is lane-local too, and P (bf16) is the B operand of that product as it stands in registers.  The key tile lies in
 // LDS as [64 keys][DKP] (main part and rotated part side by side, zero padded), the value tile transposed as [DVP][64 keys].
-#define MQ 128
+#define MQ LAT_MQ
 #define MKT 64
 template <int DKS, int NVB, bool SIG>
 __global__ __launch_bounds__(256) void latent_attn_mfma_kernel(LatAttnArgs p, int vec_ok) {
@@ -587,7 +561,10 @@ extern "C" int mi355_latent_attn(int n_seq, int max_new, int H, int hm, int D1, 
         const int vec_ok = D1 % 8 == 0 && D2 % 8 == 0 && DV % 8 == 0 && ldk1 % 8 == 0 && ldk2 % 8 == 0 && ldv % 8 == 0 && k1_hs % 8 == 0 && v_hs % 8 == 0 &&
                            ((uintptr_t)K1 & 15) == 0 && ((uintptr_t)K2 & 15) == 0 && ((uintptr_t)V & 15) == 0 &&
                            (pool == 0 || (ldp % 8 == 0 && ((uintptr_t)PK & 15) == 0 && ((uintptr_t)PV & 15) == 0));
-        if (sig_bias) launch_mfma_dk<true>(p, grid, vec_ok, ST(stream));
+        const bool o_vec = ldo % 4 == 0 && o_hs % 4 == 0 && ((uintptr_t)O & 15) == 0;
+        if (window == 0 && chunk == 0 && pool == 0 && softcap == 0.f && scale > 0.f && vec_ok && o_vec && latent_attn_full_launch(p, grid, ST(stream))) {
+            // every key j <= i, aligned rows: done
+        } else if (sig_bias) launch_mfma_dk<true>(p, grid, vec_ok, ST(stream));
         else launch_mfma_dk<false>(p, grid, vec_ok, ST(stream));
         MI355_LAUNCH_CHECK("latent_attn(mfma)");
         if (p.splits > 1) {

@@ -734,6 +734,30 @@ def diff_join(a1, a2, H, D, lam, eps, scale, gate, out_dtype):
     return out
 
 
+def diff_attn(q, k, v, H, hm, D, DV, scale, lam, eps, out_scale, gate, desc, max_new, max_keys, kv_rep):
+    """Differential attention in one kernel: q fp32 rows [H x 2 D], bf16 key rows [H / kv_rep x 2 D] and value rows [H / kv_rep x DV] (views with any pitch), both
+    maps, their difference to unit RMS per head times ``out_scale`` and the sigmoid of the fp32 ``gate`` rows (or None).  ``desc`` as in ``latent_attn``.
+    Returns bf16 [tokens, H * DV]."""
+    q_row0, n_new, past, k_row0 = desc[:4]
+    L.require_gpu(q, k, v, gate, q_row0, n_new, past, k_row0)
+    for t, n in ((q, "q"), (k, "k"), (v, "v")):
+        _rows(t, f"diff_attn({n})")
+    if q.dtype != F32 or k.dtype != BF16 or v.dtype != BF16 or (gate is not None and (gate.dtype != F32 or gate.shape[1] != H * DV or gate.stride(1) != 1)):
+        raise ValueError("diff_attn: q fp32, keys and values bf16, gate fp32 [tokens, H * DV]")
+    n_seq = q_row0.numel()
+    for t in (q_row0, n_new, past, k_row0):
+        _i32(t, "diff_attn(desc)", n_seq)
+    out = torch.empty((q.shape[0], H * DV), dtype=BF16, device=q.device)
+    splits, ws = attn_key_splits(n_seq, H // hm, max_new, 2 * hm, max_keys), None
+    if splits > 1:
+        dvp = 32 if DV <= 32 else 64 if DV <= 64 else 128 if DV <= 128 else 256
+        ws = torch.empty(n_seq * (H // hm) * -(-max_new * hm // 64) * splits * 128 * (2 + dvp), dtype=F32, device=q.device)
+    L.call("mi355_diff_attn", n_seq, int(max_new), H, hm, D, DV, L.ptr(q), q.stride(0), L.ptr(k), k.stride(0), L.ptr(v), v.stride(0), L.ptr(out), out.stride(0), L.ptr(q_row0),
+           L.ptr(n_new), L.ptr(past), L.ptr(k_row0), float(scale), int(kv_rep), splits, L.ptr(ws), 0 if ws is None else ws.numel(), float(lam), float(eps), float(out_scale),
+           L.ptr(gate), 0 if gate is None else gate.stride(0))
+    return out
+
+
 def scaled_rope_frequencies(dims, base, scaling, device):
     """fp32 [dims / 2]: base^(-2i / dims), rescaled for a longer context than the one trained on (``scaling`` = {factor, low, high, original}, or None):
     a frequency whose wavelength is shorter than original / high stays, one longer than original / low is divided by factor, between the two the
