@@ -159,9 +159,9 @@ QUERIES = {
 _lib = None
 
 
-def build(verbose=False):
-    """Compile libmi355vlm.so in-tree (hipcc --offload-arch=gfx950)."""
-    cmd = ["make", "-C", CSRC, "-j8"]
+def build(verbose=False, force=False):
+    """Compile libmi355vlm.so in-tree (hipcc --offload-arch=gfx950); ``force``: every object, also where nothing changed."""
+    cmd = ["make", "-C", CSRC, "-j8"] + (["-B"] if force else [])
     res = subprocess.run(cmd, capture_output=True, text=True)
     if res.returncode != 0:
         raise RuntimeError("building libmi355vlm.so failed:\n" + res.stdout[-4000:] + res.stderr[-4000:])
@@ -227,7 +227,9 @@ _tls = threading.local()  # .device: device of the tensors checked by this THREA
 
 
 def stream(device=None):
-    return torch.cuda.current_stream(device).cuda_stream
+    """Handle of the current HIP stream of ``device`` (None: of the current device), without the Stream object around it: launches are the bulk of a one-token step."""
+    idx = torch.cuda.current_device() if device is None or device.index is None else device.index
+    return torch._C._cuda_getCurrentRawStream(idx)
 
 
 def call(name, *args):

@@ -211,11 +211,13 @@ def test_long_prompt_then_decoding_with_dealt_out_keys(tmp_path, dt):
     model = registry.load_model(U.save(str(tmp_path), cfg, w), dt, DEV)
     toks = tokens(704, cfg["vocab"], 4)
     want = oracle(cfg, w, toks)
+    other = tokens(97, cfg["vocab"], 5)  # a shorter request beside it: most of its share of the deal is empty
+    want2 = oracle(cfg, w, other)
     b = batch_of(model)
-    got = b.step([("a", toks[:697])], [[0, 1, 350, 696]])
-    assert row_err(got, want[[0, 1, 350, 696]]) < TOL[dt]
-    got = torch.cat([b.step([("a", [t])]) for t in toks[697:]])
-    assert row_err(got, want[697:]) < TOL[dt]
+    got = b.step([("a", toks[:697]), ("b", other[:90])], [[0, 1, 350, 696], [89]])
+    assert row_err(got[:4], want[[0, 1, 350, 696]]) < TOL[dt] and row_err(got[4:], want2[89:90]) < TOL[dt]
+    got = torch.stack([b.step([("a", [t]), ("b", [u])]) for t, u in zip(toks[697:], other[90:])])
+    assert row_err(got[:, 0], want[697:]) < TOL[dt] and row_err(got[:, 1], want2[90:]) < TOL[dt]
 
 
 @pytest.mark.parametrize("dt", ["float32", "bfloat16"])
@@ -411,8 +413,39 @@ def test_attention_with_a_sink_or_without_a_softmax(dt, kind):
                 assert float((got - want).abs().max()) / ref < tol, (n, past, boost, h, extra)
 
 
+@pytest.mark.parametrize("D1,D2,DV", [(128, 0, 128), (128, 64, 128), (256, 0, 256), (256, 64, 256), (200, 0, 40), (64, 0, 200), (320, 0, 16), (32, 8, 72), (136, 40, 256)])
+def test_attention_over_every_key_at_every_width(D1, D2, DV):
+    """bf16 keys of one and of two parts (the second shared by the heads), every width class of the kernel, prompts, portions and dealt-out one-token steps, a
+    sink, fp32 and bf16 output; three sequences of unequal lengths in one launch against each alone."""
+    from llm_quest_amd import kernels_seq as S
+
+    g = torch.Generator().manual_seed(D1 + DV)
+    H, scale = 3, (D1 + D2) ** -0.5
+    sink = torch.tensor([0.5, -2.0, 2.0])
+    for new, past in (([70, 5, 129], [0, 0, 0]), ([1, 1, 1], [600, 3, 64]), ([2, 33, 1], [90, 31, 63])):
+        q = torch.randn(sum(new), H * (D1 + D2), generator=g) * 2
+        n = [a + b for a, b in zip(new, past)]
+        cap = max(n) + 4
+        k1, k2, v = (torch.randn(3 * cap, w, generator=g).to(BF16) for w in (H * D1, max(D2, 8), H * DV))
+        q_row0, row0 = [0, new[0], new[0] + new[1]], [cap * i for i in range(3)]
+        desc = tuple(dev_i32(t) for t in (q_row0, new, past, row0, row0, row0))
+        for o_dt in (F32, BF16):
+            out = torch.zeros(sum(new), H * DV, dtype=o_dt, device=DEV)
+            k1d, k2d, vd = k1.to(DEV), k2.to(DEV), v.to(DEV)
+            S.latent_attn(q.to(DEV), k1d, k2d[:, :D2] if D2 else None, vd, out, H, 1, D1, D2, DV, D1 + D2, D1, DV, DV, desc, max(new), scale, max_keys=max(n), sink=sink.to(DEV))
+            for s in range(3):
+                rows = slice(row0[s], row0[s] + n[s])
+                for h in range(H):
+                    kk = torch.cat([k1[rows, h * D1 : (h + 1) * D1], k2[rows, :D2]], dim=1).double()
+                    qq = torch.zeros(n[s], D1 + D2, dtype=F64)
+                    qq[past[s] :] = q[q_row0[s] : q_row0[s] + new[s], h * (D1 + D2) : (h + 1) * (D1 + D2)].double()
+                    want = O.softmax_map(qq, kk, v[rows, h * DV : (h + 1) * DV].double(), scale, sink[h].double())[past[s] :]
+                    got = out[q_row0[s] : q_row0[s] + new[s], h * DV : (h + 1) * DV].double().cpu()
+                    assert float((got - want).abs().max()) < 3e-2 * float(want.abs().max()), (new, past, s, h, o_dt)
+
+
 @pytest.mark.parametrize("dt", ["float32", "bfloat16"])
-@pytest.mark.parametrize("H,G,d,dv", [(4, 2, 16, 24), (3, 3, 20, 10), (6, 1, 64, 128), (2, 1, 72, 136)])
+@pytest.mark.parametrize("H,G,d,dv", [(4, 2, 16, 24), (3, 3, 20, 10), (6, 1, 64, 128), (2, 1, 72, 136), (4, 1, 128, 40), (8, 2, 32, 256)])
 def test_differential_maps_and_their_join(dt, H, G, d, dv):
     """Both maps over a cache laid out head by head as [map 1, map 2], and their join, against one softmax per map; a key far away dominant in ONE of the two
     maps only (a swapped map, or one map's key read for the other, shows)."""
