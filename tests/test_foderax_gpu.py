@@ -224,7 +224,7 @@ def test_long_prompt_then_decoding_with_dealt_out_keys(tmp_path, dt):
 def test_other_sizes_odd_and_one(tmp_path, dt):
     """Sizes that are no multiples of 8 or of each other's: one head, one key head per query head, latents of one and of odd sizes, a rotation of two entries and of
     none, no feed-forward, one expert, one group, every group kept, a recurrence of odd width, factors of 0 and 1, no cap, an embedding scale of 1, value heads
-    wider than the queries and narrower, no ``kv_heads`` entry's default in use, one layer's keys read by the next three."""
+    wider than the queries and narrower, one layer's keys read by two later ones."""
     from llm_quest_amd import registry
 
     layers = [(U.diff(heads=1, kv_heads=1, dim=6, vdim=5, rot_dims=2, base=3.0, diff=0.0), None),
