@@ -550,6 +550,11 @@ int mi355_moe_route(int64_t tokens, int E, int top, int groups, int keep, const 
                     float* wts, void* stream);
 /* Dispatch lists of `entries` = tokens * top choices: offs int32 [E + 1], perm int32 [entries] = the entries sorted by expert (token order inside one). */
 int mi355_moe_dispatch(int64_t entries, int E, const int* ids, int* offs, int* perm, void* stream);
+/* The dispatch lists of all `layers` of a step whose experts a table of the token ids picks (no router), in one launch: layer l's table int32 [vocab, top] starts
+ * at tables + meta[4 l], its top <= max_top and expert count <= max_E (<= 4096) are meta[4 l + 1] and meta[4 l + 2]; entry (t, c) belongs to expert
+ * table[tok[t], c].  Layer l's lists: offs + l * (max_E + 1) (E + 1 entries) and perm + l * tokens * max_top (tokens * top entries), as mi355_moe_dispatch writes them. */
+int mi355_moe_table_dispatch(int layers, int64_t tokens, int vocab, int max_E, int max_top, const int* tok, const int* tables, const int* meta, int* offs, int* perm,
+                             void* stream);
 /* C[b][m, n] = epi(sum_k A[b][m, k] B[b][n, k]) with general strides: A at b * a_bs + row * lda + k, B at b * b_bs + n * sbn + k * sbk (one of sbn / sbk
  * is 1), C at b * c_bs + row * ldc + n.  grp_offs (may be NULL): batch b owns the sorted rows [grp_offs[b], grp_offs[b+1]) and M bounds their number;
  * a_rows: sorted row r reads A row a_rows[r] / a_div; c_rows: it writes C row c_rows[r]; row_scale: that C row is scaled.  epi 1 = relu(x)^2.
@@ -563,8 +568,8 @@ int mi355_bgemm(int batch, int M, int N, int K, const void* A, int a_dt, int64_t
  * key j of it is K1 row k1_row0[s] + j (head stride k1_hs, D1 wide), K2 row k2_row0[s] + j (shared by heads, D2 wide), value row v_row0[s] + j.
  * Q fp32 [.., H, D1 + D2]; K1 / K2 / V of dtype dt.  A tile covers 32 / hm tokens x hm heads (hm > 1 needs k1_hs == v_hs == 0); the MFMA path (bf16,
  * D1 + D2 <= 320, DV <= 256) 128 / hm tokens, and with splits > 1 deals a tile's keys to that many workgroups whose partial results meet in ws
- * (n_seq * head tiles * token tiles * splits * 128 * (2 + DV rounded up to 32 / 64 / 128 / 256) floats).  Under a plain window (keep_first == 0) the shares start
- * at the window's lower edge, and pooled rows (below) are part of what is dealt out.
+ * (n_seq * head tiles * token tiles * splits * 128 * (2 + DV rounded up to 32 / 64 / 128 / 256) floats).  What is dealt
+ * out are the pooled rows (below), the steps that hold kept first tokens and the keys from the window's lower edge on.
  * Grouped queries: head h reads key / value head h / kv_rep (strides k1_hs / v_hs per key / value head; hm may then divide kv_rep).  window > 0: the query
  * at position i sees key j <= i only if i - j < window or j < keep_first (a sliding window that keeps the first tokens); window 0: every j <= i.
  * softcap > 0: score <- softcap * tanh(score / softcap) after the scale.  sink (fp32 [H], may be NULL): exp(sink[h]) joins head h's softmax denominator.
@@ -573,12 +578,14 @@ int mi355_bgemm(int batch, int M, int N, int K, const void* A, int a_dt, int64_t
  * dtype dt); pooled rows and tokens share one softmax.  chunk > 0: positions are cut into chunks of that many, counted from the sequence's first token,
  * and a query sees only the keys j <= i of its own chunk, floor(j / chunk) == floor(i / chunk) (no kept first tokens, no pooled blocks).
  * sig_bias (fp32 [H], may be NULL): no softmax -- a visible key's weight is sigmoid(score + sig_bias[h]), not normalised (no softcap, no sink).  o_dt: dtype
- * of the output rows O (fp32 also with bf16 keys and values). */
+ * of the output rows O (fp32 also with bf16 keys and values).  slope (fp32 [H], may be NULL): slope[h] * (i - j) is taken off the score after scale and cap (no
+ * sig_bias, no pool).  gate (fp32 rows [H x DV], pitch ldg, may be NULL): the output is multiplied element by element by sigmoid(gate). */
 int mi355_latent_attn(int n_seq, int max_new, int H, int hm, int D1, int D2, int DV, const float* Q, int64_t ldq, int q_hs, const void* K1, int64_t ldk1,
                       int k1_hs, const void* K2, int64_t ldk2, const void* V, int64_t ldv, int v_hs, void* O, int64_t ldo, int o_hs, int dt,
                       const int* q_row0, const int* n_new, const int* past, const int* k1_row0, const int* k2_row0, const int* v_row0, float scale,
                       int use_mfma, int splits, float* ws, int64_t ws_floats, int kv_rep, int window, int keep_first, float softcap, const float* sink,
-                      int pool, const void* PK, const void* PV, int64_t ldp, const int* pool_row0, int chunk, const float* sig_bias, int o_dt, void* stream);
+                      int pool, const void* PK, const void* PV, int64_t ldp, const int* pool_row0, int chunk, const float* sig_bias, int o_dt,
+                      const float* slope, const float* gate, int64_t ldg, void* stream);
 
 /* ---- parallel-sublayer hybrid decoders in ragged batches (csrc/seqrec.hip) ---- */
 /* v = x + y1[t] + sum_{p < parts} y2[t * parts + p] (fp32 rows; y1 / y2 of dtype y*_dt, may be NULL); x_out (may be NULL or x) <- v.  For each weight
@@ -597,11 +604,13 @@ int mi355_ragged_conv(int64_t tokens, int n_seq, int C, int taps, const void* x,
  * (weights qw / kw fp32 [d], NULL: none) and a rotation of their first `dims` entries (layout as mi355_rope_heads); query head h times qscale[h] (may be NULL)
  * goes to q_out fp32 [t, h * d]; key and value heads go to cache row dst_row[t] = [G x d | G x dv] of dtype c_dt.  qt_every > 0: the query at position p
  * is also multiplied by 1 + qt_coef * ln(floor((p + 1) / qt_every) + 1).  vmix (fp32 rows [G x dv], pitch ldvm, may be NULL): the cached value is
- * (1 - lam) v + lam * vmix[t].  v_heads > 0: that many value heads instead of G (rows [H x d | G x d | v_heads x dv], cache rows [G x d | v_heads x dv]). */
+ * (1 - lam) v + lam * vmix[t].  v_heads > 0: that many value heads instead of G (rows [H x d | G x d | v_heads x dv], cache rows [G x d | v_heads x dv]).
+ * unit_norm: query and key heads are divided by their root mean square (no weight).  rot_amp multiplies cosine and sine.  tie_v: src has no value rows, the
+ * values are the key rows as projected -- bias added, before norm and rotation (dv == d, G value heads). */
 int mi355_qkv_rows_append(int64_t tokens, int H, int G, int d, int dv, const void* src, int src_dt, int64_t ld_src, const float* bias, const float* qw,
                           const float* kw, float eps, const float* qscale, int dims, int layout, const float* freq, const int* pos, const int* dst_row,
                           float* q_out, int64_t ldq, void* cache, int c_dt, int64_t ldc, float qt_coef, int qt_every, const float* vmix, int64_t ldvm, float lam,
-                          int v_heads, void* stream);
+                          int v_heads, int unit_norm, float rot_amp, int tie_v, void* stream);
 /* Gated delta rule over the rows [seq_off[s], seq_off[s+1]) of each sequence, state[slot[s]] (fp32 [H, dk, dv]) read and written.  q / k rows [G * dk] (raw:
  * made unit vectors here, x / sqrt(sum x^2 + 1e-6), q also times qscale), v rows [H * dv]; value head h uses query / key head h / (H / G);
  * beta = sigmoid(b[t, h]), g = exp(-exp(A_log[h]) * softplus(a[t, h] + dt_bias[h])).  Per token: S <- g S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q.
@@ -681,6 +690,16 @@ int mi355_diff_attn(int n_seq, int max_new, int H, int hm, int D, int DV, const 
  * element (gate rows [H x D] of dtype g_dt, may be NULL). */
 int mi355_diff_join(int64_t tokens, int H, int D, const float* a1, int64_t lda1, const float* a2, int64_t lda2, float lam, float eps, float c, const void* gate, int g_dt,
                     int64_t ldg, void* out, int out_dt, int64_t ldo, void* stream);
+
+/* ---- decoders with several residual streams in ragged batches (csrc/seqhyp.hip) ---- */
+/* S streams of fp32 rows, token t's stream s at x + t * x_ts + s * x_ss (x_ss == 0: all alike).  With y (rows of dtype y_dt, `parts` per token, may be NULL):
+ * yv = y_scale * sum_p y[t * parts + p], stream to <- sum_from mix[from * S + to] x_from + put[to] * yv, all from the old streams; x_out (contiguous
+ * [tokens, S, width], may be NULL, never x) receives the streams.  read (fp32 [S], may be NULL): u = sum_s read[s] x_s of the streams as they now are; u_out (fp32, may
+ * be NULL) <- u; with w (fp32 [width]) out (dtype out_dt) <- u / sqrt(mean(u^2) + eps) * w.  rows (int64 [tokens], may be NULL): row t works on token rows[t] of x and
+ * y.  mix fp32 [S, S], put fp32 [S]. */
+int mi355_hyper_mix(int64_t tokens, int width, int S, const float* x, int64_t x_ts, int64_t x_ss, const void* y, int y_dt, int64_t ldy, int parts, float y_scale,
+                    const float* mix, const float* put, const float* read, const int64_t* rows, float* x_out, float* u_out, const float* w, float eps, void* out,
+                    int out_dt, void* stream);
 
 #ifdef __cplusplus
 }

@@ -112,12 +112,13 @@ SIGNATURES = {
     "mi355_router_logits": [_L, _I, _I, _P, _L, _P, _L, _P, _P],
     "mi355_moe_route": [_L, _I, _I, _I, _I, _P, _P, _F, _I, _P, _P, _P],
     "mi355_moe_dispatch": [_L, _I, _P, _P, _P, _P],
+    "mi355_moe_table_dispatch": [_I, _L, _I, _I, _I, _P, _P, _P, _P, _P, _P],
     "mi355_bgemm": [_I, _I, _I, _I, _P, _I, _L, _L, _P, _I, _L, _L, _L, _P, _I, _L, _L, _P, _P, _I, _P, _P, _I, _I, _P, _F, _I, _P],
-    "mi355_latent_attn": [_I, _I, _I, _I, _I, _I, _I, _P, _L, _I, _P, _L, _I, _P, _L, _P, _L, _I, _P, _L, _I, _I, _P, _P, _P, _P, _P, _P, _F, _I, _I, _P, _L, _I, _I, _I, _F, _P, _I, _P, _P, _L, _P, _I, _P, _I, _P],
+    "mi355_latent_attn": [_I, _I, _I, _I, _I, _I, _I, _P, _L, _I, _P, _L, _I, _P, _L, _P, _L, _I, _P, _L, _I, _I, _P, _P, _P, _P, _P, _P, _F, _I, _I, _P, _L, _I, _I, _I, _F, _P, _I, _P, _P, _L, _P, _I, _P, _I, _P, _P, _L, _P],
     # parallel-sublayer hybrid decoders in ragged batches (csrc/seqrec.hip)
     "mi355_group_rmsnorm_sum": [_L, _I, _P, _P, _I, _L, _P, _I, _L, _I, _P, _I, _F, _P, _P, _I, _P, _P, _P, _I, _P, _P],
     "mi355_ragged_conv": [_L, _I, _I, _I, _P, _I, _L, _P, _P, _P, _P, _P, _I, _I, _P, _I, _L, _P, _P],
-    "mi355_qkv_rows_append": [_L, _I, _I, _I, _I, _P, _I, _L, _P, _P, _P, _F, _P, _I, _I, _P, _P, _P, _P, _L, _P, _I, _L, _F, _I, _P, _L, _F, _I, _P],
+    "mi355_qkv_rows_append": [_L, _I, _I, _I, _I, _P, _I, _L, _P, _P, _P, _F, _P, _I, _I, _P, _P, _P, _P, _L, _P, _I, _L, _F, _I, _P, _L, _F, _I, _I, _F, _I, _P],
     "mi355_delta_rule_ragged": [_L, _I, _P, _P, _I, _I, _I, _I, _P, _P, _I, _L, _L, _P, _I, _L, _P, _P, _I, _L, _L, _P, _P, _F, _P, _P, _P, _P],
     "mi355_glu_rows": [_L, _I, _P, _I, _L, _I, _F, _P, _I, _L, _P],
     # decoders with sandwich norms in ragged batches (csrc/seqsand.hip)
@@ -136,6 +137,8 @@ SIGNATURES = {
     "mi355_depth_sum": [_L, _I, _P, _P, _I, _L, _F, _P, _I, _L, _F, _P, _P, _I, _L, _I, _P, _P, _L, _I, _P, _P, _P, _F, _P, _I, _P, _P],
     "mi355_diff_attn": [_I, _I, _I, _I, _I, _I, _P, _L, _P, _L, _P, _L, _P, _L, _P, _P, _P, _P, _F, _I, _I, _P, _L, _F, _F, _F, _P, _L, _P],
     "mi355_diff_join": [_L, _I, _I, _P, _L, _P, _L, _F, _F, _F, _P, _I, _L, _P, _I, _L, _P],
+    # decoders with several residual streams in ragged batches (csrc/seqhyp.hip)
+    "mi355_hyper_mix": [_L, _I, _I, _P, _L, _L, _P, _I, _L, _I, _F, _P, _P, _P, _P, _P, _P, _P, _F, _P, _I, _P],
     # measurement aid (csrc/probe.hip)
     "mi355_mfma_pipe_probe": [_I, _I, _P, _P],
     # stand-alone RoPE and dropout (csrc/rope_dropout.hip, csrc/attention_generic.hip)

@@ -19,11 +19,14 @@
 * ``DifferentialAttention`` -- two softmax maps per head over the same values, their weighted difference to unit RMS per head, a sigmoid gate per channel,
   optionally on another layer's keys and values;
 * ``MinGatedUnit``          -- a minimal gated recurrence whose gate reads the current token only, state in fp32;
-* ``GroupedSoftmaxMoE``     -- softmax-scored squared-ReLU experts chosen inside the groups with the largest members, weights not renormalised.
+* ``GroupedSoftmaxMoE``     -- softmax-scored squared-ReLU experts chosen inside the groups with the largest members, weights not renormalised;
+* ``TableMoE``              -- SiLU-gated experts that a table of the token ids picks, equal weights;
+* ``HyperConnection``       -- several residual streams: a sublayer's read-out of them, their mixing and the weights with which its output joins each.
 ``LatentAttention`` also runs without a query latent, without a rotated part, with rotate-half rotary, a sliding window, a sink in the denominator and a sigmoid output
 gate (per channel or per head); ``SlidingWindowAttention`` also
 with capped scores, a position-dependent query temperature, pooled blocks before the window, a sink in the denominator, value mixing between layers,
-chunks instead of a window, rescaled rotary frequencies, one sigmoid output gate per head and sigmoid weights without a softmax; ``SoftmaxTopkMoE`` also with a router bias, weights that are the
+chunks instead of a window, rescaled rotary frequencies (two rules), one sigmoid output gate per head or per channel, sigmoid weights without a softmax, unit-RMS queries
+and keys, a distance bias per head and values that are the unrotated keys; ``SoftmaxTopkMoE`` also with a router bias, weights that are the
 softmax over the winners alone, SiLU-gated experts and a shared expert.
 
 They run one *step* of a batch (``SeqStep``): the new tokens of every sequence, packed row after row, against what ``utils.SlotStateCache`` holds.  Inference
@@ -383,16 +386,23 @@ class SlidingWindowAttention(_Frozen):
       * ``v_mix`` ("first" / "mix") -- the first such layer of a step leaves its values for the later ones, which cache (1 - lam) v + lam v_first;
       * ``chunk`` > 0        -- instead of a window: positions are cut into chunks of that many from the sequence's first token on, i sees j <= i of its own chunk;
       * ``rot_layout`` 1     -- rotary pairs entry i with entry i + rot_dims / 2 (0: neighbours); ``rot_scaling`` {factor, low, high, original} rescales the
-        frequencies for a longer context (``kernels_seq.scaled_rope_frequencies``);
+        frequencies for a longer context (``kernels_seq.scaled_rope_frequencies``), {factor, original, fast, slow} frequencies and amplitude
+        (``kernels_seq.yarn_rope_frequencies``);
       * ``head_gate``        -- head h's output is multiplied by sigmoid(w_g h)_h, one number per head from the mixer's input, before the output projection
         (its rows follow the value rows in ``w_qkv``);
       * ``o_bias``           -- whether the output projection has a bias (default: as ``bias``);
-      * ``sigmoid``          -- no softmax: the weight of a visible key is sigmoid(score + pb[h]), ``pb`` a learned number per head, weights not normalised.
-    ``step(..., proj=rows)``: the caller has already taken the input product (with its biases) -- a mixer beside this one shares it."""
+      * ``sigmoid``          -- no softmax: the weight of a visible key is sigmoid(score + pb[h]), ``pb`` a learned number per head, weights not normalised;
+      * ``qk_norm`` "unit"   -- query and key heads are divided by their root mean square, without a weight;
+      * ``slopes``           -- one number per head: slopes[h] * (i - j) is taken off the score (after the cap) of the query at i and the key at j;
+      * ``gate``             -- the concatenated heads are multiplied element by element by the sigmoid of a projection of the mixer's input, before the output
+        projection (its rows follow the value rows in ``w_qkv``);
+      * ``tie_values``       -- no value projection: the values are the keys as projected, before norm and rotation (vdim = dim).
+    ``step(..., proj=rows)``: the caller has already taken the input product (with its biases) -- a mixer beside this one shares it.  ``step(..., cache_layer=n)``: the
+    keys and values are cache layer n's (a layer that is passed several times has rows of its own per pass)."""
 
     def __init__(self, width, heads, kv_heads, dim, vdim, scale, window, keep_first, rot_dims, rot_base, eps, layer_idx, qk_norm=True, bias=True, temp=True,
                  softcap=0.0, q_temp=None, pool=0, sink=False, v_mix=None, chunk=0, rot_layout=0, rot_scaling=None, head_gate=False, o_bias=None,
-                 sigmoid=False):
+                 sigmoid=False, slopes=None, gate=False, tie_values=False):
         super().__init__()
         if heads % kv_heads:
             raise ValueError("SlidingWindowAttention: heads must be a multiple of kv_heads")
@@ -404,18 +414,28 @@ class SlidingWindowAttention(_Frozen):
             raise ValueError("SlidingWindowAttention: v_mix is None, 'first' or 'mix'")
         if chunk and (window or keep_first or pool):
             raise ValueError("SlidingWindowAttention: chunks stand instead of a window (no kept first tokens, no pooled blocks)")
-        if sigmoid and (softcap or sink):
-            raise ValueError("SlidingWindowAttention: sigmoid weights have neither a cap nor a denominator")
+        if sigmoid and (softcap or sink or slopes):
+            raise ValueError("SlidingWindowAttention: sigmoid weights have neither a cap nor a denominator nor a distance bias")
+        if slopes is not None and (len(slopes) != heads or pool):
+            raise ValueError("SlidingWindowAttention: one slope per head; a distance bias does not combine with pooled blocks")
+        if head_gate and gate:
+            raise ValueError("SlidingWindowAttention: one gate per head or one per channel")
+        if tie_values and (vdim != dim or v_mix):
+            raise ValueError("SlidingWindowAttention: values that are the keys are as wide as they, and are not mixed")
+        if qk_norm not in (True, False, "unit"):
+            raise ValueError("SlidingWindowAttention: qk_norm is True (with weights), False or 'unit'")
+        self.unit_norm, self.slopes, self.gate, self.tie_values = qk_norm == "unit", list(slopes) if slopes is not None else None, bool(gate), bool(tie_values)
         self.chunk, self.rot_layout, self.rot_scaling, self.head_gate = int(chunk or 0), int(rot_layout), dict(rot_scaling) if rot_scaling else None, bool(head_gate)
         self.width, self.heads, self.kv_heads, self.dim, self.vdim, self.scale, self.window, self.keep_first = width, heads, kv_heads, dim, vdim, float(scale), int(window), int(keep_first)
         self.rot_dims, self.rot_base, self.eps, self.layer_idx = rot_dims, float(rot_base), float(eps), layer_idx
         self.softcap, self.q_temp, self.pool, self.v_mix = float(softcap or 0.0), (float(q_temp[0]), int(q_temp[1])) if q_temp else None, int(pool or 0), v_mix
-        n = (heads + kv_heads) * dim + kv_heads * vdim
+        n = (heads + kv_heads) * dim + (0 if tie_values else kv_heads * vdim)
         self.qkv_rows = n
-        self.w_qkv = self._param(n + (heads if head_gate else 0), width)
+        self.gate_rows = heads if head_gate else heads * vdim if gate else 0
+        self.w_qkv = self._param(n + self.gate_rows, width)
         self.b_qkv = self._param(n) if bias else None
-        self.q_norm = self._param(dim) if qk_norm else None
-        self.k_norm = self._param(dim) if qk_norm else None
+        self.q_norm = self._param(dim) if qk_norm is True else None
+        self.k_norm = self._param(dim) if qk_norm is True else None
         self.temp = self._param(heads) if temp else None
         self.sink = self._param(heads) if sink else None
         self.pb = self._param(heads) if sigmoid else None
@@ -431,7 +451,7 @@ class SlidingWindowAttention(_Frozen):
         if self.b_qkv is None:
             return None
         b = _f32(self.b_qkv)
-        return torch.cat([b, b.new_zeros(self.heads)]) if self.head_gate else b
+        return torch.cat([b, b.new_zeros(self.gate_rows)]) if self.gate_rows else b
 
     def cache_spec(self):
         spec = {"rows": self.kv_heads * (self.dim + self.vdim), "states": {}}
@@ -448,22 +468,27 @@ class SlidingWindowAttention(_Frozen):
             self.qscale = None if self.softcap else (t * self.scale).contiguous()
             if self.softcap and self.temp is not None:
                 raise ValueError("SlidingWindowAttention: a per-head temperature and a score cap do not combine")
-            self.freq = S.scaled_rope_frequencies(self.rot_dims, self.rot_base, self.rot_scaling, device) if self.rot_dims else None
+            self.slope32 = torch.tensor(self.slopes, dtype=torch.float64).to(F32).to(device) if self.slopes is not None else None
+            self.freq, self.rot_amp = None, 1.0
+            if self.rot_dims and self.rot_scaling and "fast" in self.rot_scaling:
+                self.freq, self.rot_amp = S.yarn_rope_frequencies(self.rot_dims, self.rot_base, self.rot_scaling, device)
+            elif self.rot_dims:
+                self.freq = S.scaled_rope_frequencies(self.rot_dims, self.rot_base, self.rot_scaling, device)
             self.lam32 = float(self.lam.float().item()) if self.lam is not None else 0.0
             self._ready = device
 
     @torch.no_grad()
-    def step(self, h, st, out_dtype=None, proj=None):
+    def step(self, h, st, out_dtype=None, proj=None, cache_layer=None):
         self.prepare(h.device)
         H, G, d, dv = self.heads, self.kv_heads, self.dim, self.vdim
-        L_ = self.layer_idx
+        L_ = self.layer_idx if cache_layer is None else cache_layer
         cache2d = st.cache.rows2d(L_)
         bias = self.b_qkv32
         if proj is None:
             proj = S.linear(h, self.w_qkv, out_dtype=F32)
         else:
             bias = None  # the shared product added it
-        gate = proj[:, self.qkv_rows :] if self.head_gate else None
+        gate = proj[:, self.qkv_rows :] if self.gate_rows else None
         proj = proj[:, : self.qkv_rows]
         vmix = None
         if self.v_mix == "mix":
@@ -473,7 +498,7 @@ class SlidingWindowAttention(_Frozen):
         elif self.v_mix == "first":
             st.shared["v_first"] = proj[:, (H + G) * d :]  # this step's unmixed values (a view: proj stays alive with it)
         q = S.qkv_rows_append(proj, H, G, d, dv, bias, self.q_norm32, self.k_norm32, self.eps, self.qscale, self.rot_dims, self.rot_layout, self.freq, st.pos, st.dst_row,
-                              cache2d, q_temp=self.q_temp, vmix=vmix, lam=self.lam32)
+                              cache2d, q_temp=self.q_temp, vmix=vmix, lam=self.lam32, unit_norm=self.unit_norm, rot_amp=self.rot_amp, tie_v=self.tie_values)
         pooled = row0 = None
         if self.pool:
             p2d = st.cache.pooled2d(L_)
@@ -484,7 +509,8 @@ class SlidingWindowAttention(_Frozen):
         hm = _largest_pow2_divisor(H // G)
         S.latent_attn(q, cache2d, None, cache2d[:, G * d :], ctx, H, hm, d, 0, dv, d, d, dv, dv, (st.q_row0, st.n_new, st.past, st.cache_row0, st.cache_row0, st.cache_row0),
                       st.max_new, self.scale if self.softcap else 1.0, max_keys=st.max_keys, kv_rep=H // G, window=self.window, keep_first=self.keep_first,
-                      softcap=self.softcap, sink=self.sink32, pool=self.pool, pooled=pooled, pool_row0=row0, chunk=self.chunk, sig_bias=self.pb32)
+                      softcap=self.softcap, sink=self.sink32, pool=self.pool, pooled=pooled, pool_row0=row0, chunk=self.chunk, sig_bias=self.pb32,
+                      slope=self.slope32, gate=gate if self.gate else None)
         if self.head_gate:
             ctx = S.unary_rows(ctx, S.UNARY_HEAD_GATE, gate=gate, group=dv)
         return S.linear(ctx, self.w_o, bias=self.b_o32, out_dtype=out_dtype)
@@ -550,25 +576,14 @@ class GatedMLP(_Frozen):
         return S.linear(S.glu_rows(S.linear(h, self.w_gate_up), self.act), self.w_down, out_dtype=out_dtype)
 
 
-class SoftmaxTopkMoE(_Frozen):
-    """``experts`` gated feed-forward experts without biases, ``top`` per token.  Router: fp32 logits, softmax over ALL experts, the ``top`` largest scores
-    win and ARE the weights (not renormalised).  Expert: g = min(gate x, limit), u = clamp(up x, -limit, limit), down(g sigmoid(1.702 g) (u + 1)).
-    Returns the weighted outputs as ``top`` fp32 rows per token; the sum is taken by the residual kernel that follows.  Options: ``act`` "silu": the expert is
-    down(silu(gate x) (up x)); ``router_bias``: a bias on the router's logits; ``chosen_softmax``: the weights are the softmax over the winners' logits alone;
-    ``shared_ff`` > 0: a dense expert of the same form (``self.shared``) that every token uses -- ``step`` then returns (expert rows, shared rows [T, width])."""
+class GatedExperts(_Frozen):
+    """``experts`` gated feed-forward experts without biases, ``top`` per token, whoever picks them.  ``act`` "silu": down(silu(gate x) (up x)); "clamped": g = min(gate x,
+    limit), u = clamp(up x, -limit, limit), down(g sigmoid(1.702 g) (u + 1)).  The gated activation is the epilogue of the gate-up product."""
 
-    def __init__(self, width, ff, experts, top, limit=0.0, act="clamped", router_bias=False, chosen_softmax=False, shared_ff=0):
-        super().__init__()
+    def _expert_params(self, width, ff, experts, top, limit, act):
         if act not in ("clamped", "silu"):
-            raise ValueError("SoftmaxTopkMoE: act is 'clamped' or 'silu'")
-        self.width, self.ff, self.experts, self.top, self.limit = width, ff, experts, top, float(limit)
-        self.act, self.chosen_softmax = act, bool(chosen_softmax)
-        self.b_router = self._param(experts) if router_bias else None
-        if shared_ff and act != "silu":
-            raise ValueError("SoftmaxTopkMoE: the shared expert comes with SiLU-gated experts")
-        self.shared = GatedMLP(width, shared_ff, act=S.GLU_SILU) if shared_ff else None
-        self._ready = None
-        self.w_router = self._param(experts, width)
+            raise ValueError("gated experts: act is 'clamped' or 'silu'")
+        self.width, self.ff, self.experts, self.top, self.limit, self.act = width, ff, experts, top, float(limit), act
         self.w_gate_up = self._param(experts, 64 * (-(-ff // 32)), width)  # per expert S.pack_gate_up(gate, up): [32 gate rows | 32 up rows] blocks
         self.w_down = self._param(experts, width, ff)
 
@@ -577,10 +592,40 @@ class SoftmaxTopkMoE(_Frozen):
         self.w_gate_up.data.copy_(torch.stack([S.pack_gate_up(g, u) for g, u in zip(gates, ups)]))
         self.w_down.data.copy_(torch.stack(list(downs)))
 
+    def run_experts(self, h, offs, perm, wts=None):
+        """h [T, width] through the experts of the dispatch lists -> fp32 [T * top, width], each row times its weight (None: 1)."""
+        T, E, top, ff = h.shape[0], self.experts, self.top, self.ff
+        np_ = self.w_gate_up.shape[1]
+        act = torch.empty((T * top, ff), dtype=h.dtype, device=h.device)
+        S.bgemm(h, self.w_gate_up, act, T * top, np_, self.width, batch=E, sbn=self.width, b_bs=np_ * self.width, grp_offs=offs, a_rows=perm, a_div=top,
+                epi=S.EPI_SILU_GLU if self.act == "silu" else S.EPI_CLAMPED_SWISH_GLU, limit=self.limit, n_out=ff)
+        out = torch.empty((T * top, self.width), dtype=F32, device=h.device)
+        S.bgemm(act, self.w_down, out, T * top, self.width, ff, batch=E, sbn=ff, b_bs=self.width * ff, grp_offs=offs, c_rows=perm, row_scale=None if wts is None else wts.view(-1))
+        return out
+
+
+class SoftmaxTopkMoE(GatedExperts):
+    """``experts`` gated feed-forward experts without biases, ``top`` per token.  Router: fp32 logits, softmax over ALL experts, the ``top`` largest scores
+    win and ARE the weights (not renormalised).  Expert: g = min(gate x, limit), u = clamp(up x, -limit, limit), down(g sigmoid(1.702 g) (u + 1)).
+    Returns the weighted outputs as ``top`` fp32 rows per token; the sum is taken by the residual kernel that follows.  Options: ``act`` "silu": the expert is
+    down(silu(gate x) (up x)); ``router_bias``: a bias on the router's logits; ``chosen_softmax``: the weights are the softmax over the winners' logits alone;
+    ``shared_ff`` > 0: a dense expert of the same form (``self.shared``) that every token uses -- ``step`` then returns (expert rows, shared rows [T, width])."""
+
+    def __init__(self, width, ff, experts, top, limit=0.0, act="clamped", router_bias=False, chosen_softmax=False, shared_ff=0):
+        super().__init__()
+        self.chosen_softmax = bool(chosen_softmax)
+        self.b_router = self._param(experts) if router_bias else None
+        if shared_ff and act != "silu":
+            raise ValueError("SoftmaxTopkMoE: the shared expert comes with SiLU-gated experts")
+        self.shared = GatedMLP(width, shared_ff, act=S.GLU_SILU) if shared_ff else None
+        self._ready = None
+        self.w_router = self._param(experts, width)
+        self._expert_params(width, ff, experts, top, limit, act)
+
     @torch.no_grad()
     def step(self, h32, h):
         """h32: the normed fp32 rows (the router reads them), h: the same rows in the activation dtype -> fp32 [T * top, width]."""
-        T, E, top, ff = h.shape[0], self.experts, self.top, self.ff
+        E, top = self.experts, self.top
         if self._ready != h.device:
             self.b_router32 = _f32(self.b_router)
             self._ready = h.device
@@ -592,15 +637,86 @@ class SoftmaxTopkMoE(_Frozen):
                 raise ValueError("SoftmaxTopkMoE: a router bias comes with weights over the winners")
             ids, wts = S.moe_route(logits, None, top, 1, 1, 1.0, softmax=True)
         offs, perm = S.moe_dispatch(ids.view(-1), E)
-        np_ = self.w_gate_up.shape[1]
-        act = torch.empty((T * top, ff), dtype=h.dtype, device=h.device)  # the gated activation is the gate-up product's epilogue
-        S.bgemm(h, self.w_gate_up, act, T * top, np_, self.width, batch=E, sbn=self.width, b_bs=np_ * self.width, grp_offs=offs, a_rows=perm, a_div=top,
-                epi=S.EPI_SILU_GLU if self.act == "silu" else S.EPI_CLAMPED_SWISH_GLU, limit=self.limit, n_out=ff)
-        out = torch.empty((T * top, self.width), dtype=F32, device=h.device)
-        S.bgemm(act, self.w_down, out, T * top, self.width, ff, batch=E, sbn=ff, b_bs=self.width * ff, grp_offs=offs, c_rows=perm, row_scale=wts.view(-1))
+        out = self.run_experts(h, offs, perm, wts)
         if self.shared is not None:
             return out, self.shared.step(h32, h, out_dtype=F32)
         return out
+
+
+class TableMoE(GatedExperts):
+    """SiLU-gated experts without a router: ``table`` (int32 [vocab, top], the entries of a row differ) gives every token id its experts, each with weight 1 / top.
+    The lists of all such layers of a step are made in one launch (``dispatch``); ``step`` returns the experts' rows [T * top, width] unweighted -- the kernel
+    that adds them to the stream applies 1 / top."""
+
+    def __init__(self, width, ff, experts, top, vocab):
+        super().__init__()
+        if not 1 <= top <= experts:
+            raise ValueError("TableMoE: a token uses between one and all of the experts")
+        self.vocab = int(vocab)
+        self._expert_params(width, ff, experts, top, 0.0, "silu")
+        self.register_buffer("table", torch.arange(top, dtype=I32).repeat(vocab, 1))
+
+    def load_table(self, table):
+        if tuple(table.shape) != tuple(self.table.shape) or table.is_floating_point():
+            raise ValueError(f"TableMoE: the table is integers {tuple(self.table.shape)}, got {table.dtype} {tuple(table.shape)}")
+        if int(table.min()) < 0 or int(table.max()) >= self.experts:
+            raise ValueError("TableMoE: the table names an expert that does not exist")
+        s = table.sort(dim=1).values
+        if bool((s[:, 1:] == s[:, :-1]).any()):
+            raise ValueError("TableMoE: a row of the table names an expert twice")
+        self.table.copy_(table)
+
+    @staticmethod
+    def gather_tables(layers):
+        """What ``dispatch`` needs of the given layers, made once per model and device: (tables one after the other, their descriptors, [(top, experts)], vocab)."""
+        meta, at = [], 0
+        for m in layers:
+            meta += [at, m.top, m.experts, 0]
+            at += m.table.numel()
+        if at >= 1 << 31:
+            raise ValueError("TableMoE: the tables of all layers together hold at most 2^31 entries")
+        dev = layers[0].table.device
+        return torch.cat([m.table.reshape(-1) for m in layers]), torch.tensor(meta, dtype=I32).to(dev), [(m.top, m.experts) for m in layers], layers[0].vocab
+
+    @staticmethod
+    def dispatch(gathered, st):
+        """Every layer's dispatch lists for the step's tokens: [(offs, perm)] in the order of ``gather_tables``."""
+        tables, meta, specs, vocab = gathered
+        return S.moe_table_dispatch(st.tok, vocab, tables, meta, specs)
+
+    @torch.no_grad()
+    def step(self, h, lists):
+        return self.run_experts(h, *lists)
+
+
+class HyperConnection(_Frozen):
+    """One sublayer's weights on ``streams`` parallel residual streams: its input is sum_s read[s] x_s; with its output y stream t becomes
+    sum_s mix[s, t] x_s + put[t] y (``kernels_seq.hyper_mix`` takes both, the join of one sublayer together with the read-out of the next)."""
+
+    def __init__(self, streams):
+        super().__init__()
+        self.read, self.put, self.mix = self._param(streams), self._param(streams), self._param(streams, streams)
+        self._ready = None
+
+    def prepare(self, device):
+        if self._ready != device:
+            self.read32, self.put32, self.mix32 = _f32(self.read), _f32(self.put), _f32(self.mix)
+            self._ready = device
+
+
+def geometric_slopes(heads):
+    """The distance-bias slope of every head: 2^(-8 (h + 1) / heads)."""
+    return [2.0 ** (-8.0 * (h + 1) / heads) for h in range(heads)]
+
+
+def layer_runs(n_layers, loop):
+    """The layers of a stack in the order they run: ``loop`` = {start, stop, times}: layers start .. stop-1 run ``times`` times in a row with the same weights."""
+    if not loop:
+        return list(range(n_layers))
+    a, b, n = int(loop["start"]), int(loop["stop"]), int(loop["times"])
+    if not (0 <= a <= b <= n_layers and n >= 1):
+        raise ValueError(f"loop: layers {a} .. {b} x {n} of {n_layers}")
+    return list(range(a)) + list(range(a, b)) * n + list(range(b, n_layers))
 
 
 class ActMLP(_Frozen):

@@ -29,7 +29,30 @@ struct LatAttnArgs {
     const int* pool_row0;
     const float* sig_bias;  // fp32 [H] or NULL: weights sigmoid(score + sig_bias[head]) instead of a softmax
     int o_dt;               // dtype of the output rows (MI355_DT_*)
+    const float* slope;     // fp32 [H] or NULL: slope[head] * (i - j) is taken off the (scaled, capped) score of query position i and key j
+    const float* gate;      // fp32 rows [H x DV] or NULL: the output is multiplied element by element by sigmoid(gate)
+    int64_t ldg;
 };
+
+// keys below this one are seen by no row of a tile whose first row stands at position pos0, kept first tokens aside (rows of a tile are consecutive positions)
+__device__ __forceinline__ int tile_key_floor(int pos0, int window, int chunk) {
+    const int w = window > 0 ? pos0 - window + 1 : 0, c = chunk > 0 ? pos0 / chunk * chunk : 0;
+    return max(w, c);
+}
+// The 64-key steps a tile walks: those that hold kept first tokens below the tile's window, then everything from the window's lower edge to the last key.
+struct KeySteps {
+    int keep, key_lo, n;  // steps of kept tokens; first key of the others; all steps
+    __device__ __forceinline__ int key(int v) const { return v < keep ? v * 64 : key_lo + (v - keep) * 64; }
+};
+__device__ __forceinline__ KeySteps key_steps(int pos0, int n_keys, int window, int keep_first, int chunk) {
+    const int lo = max(tile_key_floor(pos0, window, chunk), 0) / 64;
+    KeySteps k;
+    k.keep = min((keep_first + 63) / 64, lo);
+    k.key_lo = lo * 64;
+    k.n = k.keep + (n_keys - k.key_lo + 63) / 64;
+    return k;
+}
+__device__ __forceinline__ float gate_of(float g) { return 1.0f / (1.0f + expf(-g)); }
 
 // Launches the kernel for attention over every key j <= i (no window, chunk, pooled rows or cap; scale > 0; rows 16-byte aligned, widths multiples of 8) if it
 // holds these sizes; false: the caller takes the general kernel.  Partial results under key splits have the general kernel's layout.

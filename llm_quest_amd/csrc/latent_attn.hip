@@ -10,7 +10,8 @@
 // only enters the softmax denominator, and POOLED blocks in front of a window -- one mean key / value row per `pool` tokens, kept by the caller in a
 // second buffer; the query at position i sees block b iff all of its tokens have left the window, (b + 1) pool <= i - window + 1.  Pooled rows
 // and tokens share one softmax: the key loop simply runs over the pooled rows first.  Without a softmax (sig_bias): the weight of a visible key is
-// sigmoid(score + sig_bias[head]), not normalised -- no running maximum, no rescaling, no denominator.
+// sigmoid(score + sig_bias[head]), not normalised -- no running maximum, no rescaling, no denominator.  A per-head distance bias (slope) is taken off the
+// score after the cap; a sigmoid gate per output element (gate) multiplies the result.
 // Scores, softmax statistics and the output accumulators are fp32.  A tile is `tm` tokens x `hm` heads = 32 query rows (hm > 1 only with shared
 // keys and values) against 64 keys at a time.
 //
@@ -31,11 +32,6 @@ __device__ __forceinline__ float cap_score(float s, float cap) { return cap > 0.
 // key j for the query at position lim (lim < 0: a padding row that sees nothing)
 __device__ __forceinline__ bool key_visible(int j, int lim, int window, int keep_first, int chunk) {
     return j <= lim && (window <= 0 || lim - j < window || j < keep_first) && (chunk <= 0 || j >= lim / chunk * chunk);
-}
-// keys below this one are seen by no row of a tile whose first row stands at position pos0 (rows of a tile are consecutive positions)
-__device__ __forceinline__ int tile_key_floor(int pos0, int window, int chunk) {
-    const int w = window > 0 ? pos0 - window + 1 : 0, c = chunk > 0 ? pos0 / chunk * chunk : 0;
-    return max(w, c);
 }
 
 __device__ __forceinline__ float lda_dt(const void* p, int dt, int64_t i) { return dt == MI355_DT_F32 ? ((const float*)p)[i] : bf2f(((const bf16_t*)p)[i]); }
@@ -82,6 +78,11 @@ __global__ __launch_bounds__(256) void latent_attn_fma_kernel(LatAttnArgs p) {
     int npv[2];
 #pragma unroll
     for (int a = 0; a < 2; ++a) npv[a] = p.pool > 0 ? pooled_visible(lim[a], p.window, p.pool) : 0;
+    float sl[2] = {0.f, 0.f};  // the rows' distance slopes
+    if (p.slope) {
+#pragma unroll
+        for (int a = 0; a < 2; ++a) sl[a] = p.slope[min(head0 + (2 * ty + a) % p.hm, p.H - 1)];
+    }
     float sb[2] = {0.f, 0.f};  // the rows' biases of the sigmoid weights
     if (p.sig_bias) {
 #pragma unroll
@@ -135,7 +136,7 @@ __global__ __launch_bounds__(256) void latent_attn_fma_kernel(LatAttnArgs p) {
             for (int i = 0; i < 4; ++i) {
                 const int j = j0 + tx + 16 * i;
                 const bool vis = seg ? j < npv[a] : key_visible(j, lim[a], p.window, p.keep_first, p.chunk);
-                acc[a][i] = vis ? cap_score(acc[a][i] * p.scale, p.softcap) : -__builtin_huge_valf();
+                acc[a][i] = vis ? cap_score(acc[a][i] * p.scale, p.softcap) - sl[a] * (float)(lim[a] - j) : -__builtin_huge_valf();
                 mx = fmaxf(mx, acc[a][i]);
             }
 #pragma unroll
@@ -206,7 +207,8 @@ __global__ __launch_bounds__(256) void latent_attn_fma_kernel(LatAttnArgs p) {
         for (int i = 0; i < NC; ++i) {
             const int col = c + 64 * i;
             if (col >= p.DV) continue;
-            const float v = o[r][i] * inv;
+            float v = o[r][i] * inv;
+            if (p.gate) v *= gate_of(p.gate[(qr0 + tok) * p.ldg + (int64_t)head * p.DV + col]);
             if (p.o_dt == MI355_DT_F32) ((float*)p.O)[ob + col] = v;
             else ((bf16_t*)p.O)[ob + col] = f2bf(v);
         }
@@ -258,13 +260,12 @@ __global__ __launch_bounds__(256) void latent_attn_mfma_kernel(LatAttnArgs p, in
         }
     }
     const int n_keys = past + min(tok0 + tm, n_new);
-    const int win_lo = tile_key_floor(past + tok0, p.window, p.chunk);  // keys below it are outside the window (or chunk) of every row of the tile
-    // The tile's work is a list of 64-row steps: first the pooled rows any of its rows may see, then the keys from key_lo on (under a plain window dealt
-    // out to several workgroups that is the window's lower edge, else 0: steps below a window are skipped one by one).  Workgroup `split` takes its share.
+    // The tile's work is a list of 64-row steps: first the pooled rows any of its rows may see, then its key steps (kept first tokens, the window).
+    // Workgroup `split` takes its share.
     const int n_pool = p.pool > 0 ? pooled_visible(n_keys - 1, p.window, p.pool) : 0;
     const int pool_steps = (n_pool + MKT - 1) / MKT;
-    const int key_lo = (p.splits > 1 && p.keep_first == 0 && win_lo > 0) ? win_lo / MKT * MKT : 0;
-    const int all_steps = pool_steps + (n_keys - key_lo + MKT - 1) / MKT;
+    const KeySteps ks = key_steps(past + tok0, n_keys, p.window, p.keep_first, p.chunk);
+    const int all_steps = pool_steps + ks.n;
     int v_lo = 0, v_hi = all_steps;
     if (p.splits > 1) {
         const int per = (all_steps + p.splits - 1) / p.splits;
@@ -288,12 +289,12 @@ __global__ __launch_bounds__(256) void latent_attn_mfma_kernel(LatAttnArgs p, in
     const int npv = p.pool > 0 ? pooled_visible(lim, p.window, p.pool) : 0;  // the pooled rows this lane's query sees
     const int64_t pr0 = p.pool > 0 ? p.pool_row0[s] : 0;
     const float capl = p.softcap * 1.4426950408889634f;
+    const float sl2 = !SIG && p.slope ? p.slope[row_ok ? head : 0] * 1.4426950408889634f : 0.f;
     const float sgb = SIG ? p.sig_bias[row_ok ? head : 0] * 1.4426950408889634f : 0.f;
     for (int v = v_lo; v < v_hi; ++v) {
         const bool seg = v < pool_steps;  // the pooled rows come first
-        const int j0 = seg ? v * MKT : key_lo + (v - pool_steps) * MKT;
+        const int j0 = seg ? v * MKT : ks.key(v - pool_steps);
         const int n_here = seg ? n_pool : n_keys;
-        if (!seg && j0 + MKT <= win_lo && j0 >= p.keep_first) continue;  // block-uniform: no row sees a key of this step
         const bf16_t* Kp = seg ? (const bf16_t*)p.PK : K1;
         const bf16_t* Vp = seg ? (const bf16_t*)p.PV : V;
         const int64_t kr = seg ? pr0 : k1r0, vr = seg ? pr0 : vr0, ldk = seg ? p.ldp : p.ldk1, ldvv = seg ? p.ldp : p.ldv;
@@ -377,7 +378,7 @@ __global__ __launch_bounds__(256) void latent_attn_mfma_kernel(LatAttnArgs p, in
                 for (int r = 0; r < 16; ++r) {
                     const int j = j0 + kb * 32 + 8 * (r >> 2) + 4 * hf + (r & 3);
                     const bool vis = seg ? j < npv : (key_visible(j, lim, p.window, p.keep_first, p.chunk) && j < n_keys);
-                    const float v = !vis ? NEG : (p.softcap > 0.f ? capl * tanhf(sacc[kb][r] * p.scale / p.softcap) : sacc[kb][r] * sc2);
+                    const float v = !vis ? NEG : (p.softcap > 0.f ? capl * tanhf(sacc[kb][r] * p.scale / p.softcap) : sacc[kb][r] * sc2) - sl2 * (float)(lim - j);
                     sacc[kb][r] = v;
                     mx = fmaxf(mx, v);
                 }
@@ -433,6 +434,16 @@ __global__ __launch_bounds__(256) void latent_attn_mfma_kernel(LatAttnArgs p, in
         inv = f / (l_run * f + exp2f(sk - m2));
     }
     const int64_t o0 = (qr0 + tok) * p.ldo + (int64_t)head * p.o_hs;
+    if (p.gate) {
+        const float* g = p.gate + (qr0 + tok) * p.ldg + (int64_t)head * p.DV;
+#pragma unroll
+        for (int vb = 0; vb < NVB; ++vb)
+#pragma unroll
+            for (int r = 0; r < 16; ++r) {
+                const int dv = vb * 32 + 8 * (r >> 2) + 4 * hf + (r & 3);
+                if (dv < p.DV) oacc[vb][r] *= gate_of(g[dv]);
+            }
+    }
     if (p.o_dt == MI355_DT_F32) {
         float* orow = (float*)p.O + o0;
 #pragma unroll
@@ -488,7 +499,8 @@ __global__ __launch_bounds__(256) void latent_attn_combine_kernel(LatAttnArgs p,
             if (p.sig_bias) acc += w;  // sigmoid weights simply add up
             else if (mi != -__builtin_huge_valf()) acc += w * exp2f(mi - m);
         }
-        const float v = p.sig_bias ? acc : acc / l;
+        float v = p.sig_bias ? acc : acc / l;
+        if (p.gate) v *= gate_of(p.gate[((int64_t)p.q_row0[s] + tok) * p.ldg + (int64_t)head * p.DV + dv]);
         if (p.o_dt == MI355_DT_F32) ((float*)p.O)[o0 + dv] = v;
         else ((bf16_t*)p.O)[o0 + dv] = f2bf(v);
     }
@@ -515,7 +527,8 @@ extern "C" int mi355_latent_attn(int n_seq, int max_new, int H, int hm, int D1, 
                                  int k1_hs, const void* K2, int64_t ldk2, const void* V, int64_t ldv, int v_hs, void* O, int64_t ldo, int o_hs, int dt,
                                  const int* q_row0, const int* n_new, const int* past, const int* k1_row0, const int* k2_row0, const int* v_row0, float scale,
                                  int use_mfma, int splits, float* ws, int64_t ws_floats, int kv_rep, int window, int keep_first, float softcap, const float* sink,
-                                 int pool, const void* PK, const void* PV, int64_t ldp, const int* pool_row0, int chunk, const float* sig_bias, int o_dt, void* stream) {
+                                 int pool, const void* PK, const void* PV, int64_t ldp, const int* pool_row0, int chunk, const float* sig_bias, int o_dt, const float* slope,
+                                 const float* gate, int64_t ldg, void* stream) {
     MI355_REQUIRE(n_seq > 0 && n_seq <= 65535 && max_new > 0 && H > 0 && D1 > 0 && D2 >= 0 && DV > 0 && DV <= 512 && Q && K1 && V && O && (D2 == 0 || K2),
                   "latent_attn: bad arguments (value width <= 512)");
     MI355_REQUIRE(dt == MI355_DT_BF16 || dt == MI355_DT_F32, "latent_attn: bad dtype");
@@ -530,6 +543,8 @@ extern "C" int mi355_latent_attn(int n_seq, int max_new, int H, int hm, int D1, 
                   "latent_attn: pooled blocks need a window, one-part keys and the pooled rows (laid out like the key / value rows)");
     MI355_REQUIRE(o_dt == MI355_DT_BF16 || o_dt == MI355_DT_F32, "latent_attn: bad output dtype");
     MI355_REQUIRE(!sig_bias || (softcap == 0.f && !sink), "latent_attn: sigmoid weights combine with neither a cap nor a sink");
+    MI355_REQUIRE(!slope || (!sig_bias && pool == 0), "latent_attn: a distance bias combines with neither sigmoid weights nor pooled blocks");
+    MI355_REQUIRE(!gate || ldg >= (int64_t)H * DV, "latent_attn: the gate's rows hold one entry per output");
     MI355_REQUIRE(q_row0 && n_new && past && k1_row0 && k2_row0 && v_row0, "latent_attn: sequence descriptors missing");
     MI355_REQUIRE(ldq >= (int64_t)(H - 1) * q_hs + D1 + D2 && ldo >= (int64_t)(H - 1) * o_hs + DV && ldk1 >= (int64_t)((H - 1) / kv_rep) * k1_hs + D1 && ldv >= (int64_t)((H - 1) / kv_rep) * v_hs + DV &&
                       (D2 == 0 || ldk2 >= D2),
@@ -545,6 +560,7 @@ extern "C" int mi355_latent_attn(int n_seq, int max_new, int H, int hm, int D1, 
     p.softcap = softcap, p.sink = sink, p.pool = pool, p.PK = PK, p.PV = PV, p.ldp = ldp, p.pool_row0 = pool_row0;
     p.splits = 1, p.ws = nullptr;
     p.sig_bias = sig_bias, p.o_dt = o_dt;
+    p.slope = slope, p.gate = gate, p.ldg = ldg;
     const bool mfma = use_mfma && D1 + D2 <= 320 && DV <= 256;  // what the MFMA kernel keeps in registers; larger heads take the FMA path
     const int tm = (mfma ? MQ : AM) / hm;
     const int64_t gx = ((int64_t)max_new + tm - 1) / tm, gy = (H + hm - 1) / hm;
@@ -562,7 +578,7 @@ extern "C" int mi355_latent_attn(int n_seq, int max_new, int H, int hm, int D1, 
                            ((uintptr_t)K1 & 15) == 0 && ((uintptr_t)K2 & 15) == 0 && ((uintptr_t)V & 15) == 0 &&
                            (pool == 0 || (ldp % 8 == 0 && ((uintptr_t)PK & 15) == 0 && ((uintptr_t)PV & 15) == 0));
         const bool o_vec = ldo % 4 == 0 && o_hs % 4 == 0 && ((uintptr_t)O & 15) == 0;
-        if (window == 0 && chunk == 0 && pool == 0 && softcap == 0.f && scale > 0.f && vec_ok && o_vec && latent_attn_full_launch(p, grid, ST(stream))) {
+        if (window == 0 && chunk == 0 && pool == 0 && softcap == 0.f && !slope && !gate && scale > 0.f && vec_ok && o_vec && latent_attn_full_launch(p, grid, ST(stream))) {
             // every key j <= i, aligned rows: done
         } else if (sig_bias) launch_mfma_dk<true>(p, grid, vec_ok, ST(stream));
         else launch_mfma_dk<false>(p, grid, vec_ok, ST(stream));

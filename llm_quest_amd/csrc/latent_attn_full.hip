@@ -20,8 +20,6 @@ struct DiffJoinArgs {  // the join of two maps: o = a1 - lam a2, o / sqrt(mean(o
     float lam, eps, c;
 };
 
-__device__ __forceinline__ float gate_of(float g) { return 1.0f / (1.0f + expf(-g)); }
-
 template <int DKS, int NVB, bool SIG, int MAPS>
 __global__ __launch_bounds__(256, NVB <= 4 && DKS * MAPS <= 16 ? 2 : 1) void latent_attn_full_kernel(LatAttnArgs p, DiffJoinArgs dj) {
     constexpr int DKP = DKS * 16, KROW = MAPS * DKP, DVP = NVB * 32, KLD = KROW + 8, VLD = DVP == 32 ? 32 : DVP + 32;

@@ -700,44 +700,118 @@ extern "C" int mi355_moe_route(int64_t tokens, int E, int top, int groups, int k
 }
 
 // Dispatch lists: entries (token, choice) sorted by expert.  offs[e] .. offs[e+1] are expert e's rows of `perm`, perm[r] = token * top + choice.
-// One workgroup: histogram in LDS, scan, then positions in token order (rows of an expert stay in token order: a fixed layout, no atomics).
-__global__ __launch_bounds__(1024) void moe_dispatch_kernel(int64_t n, int E, const int* __restrict__ ids, int* __restrict__ offs, int* __restrict__ perm) {
-    extern __shared__ int cnt[];  // [E + 1] counts, then running offsets
-    for (int e = threadIdx.x; e <= E; e += blockDim.x) cnt[e] = 0;
+// One workgroup, a counting sort that keeps token order inside an expert (a fixed layout): wave w owns the w-th run of entries and a row of counters in LDS; counts,
+// a prefix over (expert, wave), then every wave places its entries 64 at a time -- lanes of the same expert find each other by one ballot per bit of the expert's
+// number.  The first DISP_U x 64 entries of a wave stay in registers between the two passes.  id_of(i): the expert of entry i (outside [0, E): no expert).
+#define DISP_U 16
+#define DISP_COUNTERS 15360
+static inline int disp_waves(int E) { return DISP_COUNTERS / E < 16 ? (DISP_COUNTERS / E < 1 ? 1 : DISP_COUNTERS / E) : 16; }
+template <typename IdOf>
+__device__ __forceinline__ void dispatch_lists(int64_t n, int E, int nw, IdOf id_of, int* __restrict__ offs, int* __restrict__ perm, int* lds) {
+    volatile int* cnt = lds;          // [nw][E]
+    int* part = lds + nw * E;         // [16] totals of the waves' scans
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    const int64_t per = ((n + nw - 1) / nw + 63) / 64 * 64;
+    const int64_t lo = wave < nw ? min((int64_t)wave * per, n) : n, hi = wave < nw ? min(lo + per, n) : n;
+    int ids[DISP_U];
+    auto fetch = [&](int64_t i0) {
+#pragma unroll
+        for (int u = 0; u < DISP_U; ++u) {
+            const int64_t i = i0 + 64 * u + lane;
+            const int e = i < hi ? id_of(i) : -1;
+            ids[u] = (unsigned)e < (unsigned)E ? e : -1;
+        }
+    };
+    for (int i = threadIdx.x; i < nw * E; i += 1024) cnt[i] = 0;
     __syncthreads();
-    for (int64_t i = threadIdx.x; i < n; i += blockDim.x) {
-        const int e = ids[i];
-        if (e >= 0 && e < E) atomicAdd(&cnt[e], 1);
+    for (int64_t i0 = lo; i0 < hi; i0 += 64 * DISP_U) {
+        fetch(i0);
+#pragma unroll
+        for (int u = 0; u < DISP_U; ++u)
+            if (ids[u] >= 0) atomicAdd(&lds[wave * E + ids[u]], 1);
     }
     __syncthreads();
-    if (threadIdx.x == 0) {
-        int run = 0;
-        for (int e = 0; e < E; ++e) {
-            const int c = cnt[e];
-            cnt[e] = run;
-            offs[e] = run;
+    // thread t owns `own` neighbouring experts: their totals, a scan over the workgroup, then the start of every (expert, wave)
+    const int own = (E + 1023) / 1024, e0 = threadIdx.x * own, e1 = min(e0 + own, E);
+    int sum = 0;
+    for (int e = e0; e < e1; ++e)
+        for (int w = 0; w < nw; ++w) sum += cnt[w * E + e];
+    int incl = sum;
+    for (int o = 1; o < 64; o <<= 1) {
+        const int v = __shfl_up(incl, o, 64);
+        if (lane >= o) incl += v;
+    }
+    if (lane == 63) part[wave] = incl;
+    __syncthreads();
+    int run = incl - sum;
+    for (int w = 0; w < wave; ++w) run += part[w];
+    for (int e = e0; e < e1; ++e) {
+        offs[e] = run;
+        for (int w = 0; w < nw; ++w) {
+            const int c = cnt[w * E + e];
+            cnt[w * E + e] = run;
             run += c;
         }
-        offs[E] = run;
     }
+    if (e0 < E && e1 == E) offs[E] = run;
     __syncthreads();
-    // wave e walks the entries 64 at a time and places its expert's rows by ballot + prefix count
-    const int lane = threadIdx.x & 63, nw = blockDim.x >> 6;
-    for (int e = threadIdx.x >> 6; e < E; e += nw) {
-        int at = cnt[e];
-        for (int64_t i0 = 0; i0 < n; i0 += 64) {
-            const int64_t i = i0 + lane;
-            const bool m = i < n && ids[i] == e;
-            const unsigned long long b = __ballot(m);
-            if (m) perm[at + __popcll(b & ((1ull << lane) - 1ull))] = (int)i;
-            at += __popcll(b);
+    int bits = 0;
+    while ((1 << bits) < E) ++bits;
+    for (int64_t i0 = lo; i0 < hi; i0 += 64 * DISP_U) {
+        if (hi - lo > 64 * DISP_U) fetch(i0);
+#pragma unroll
+        for (int u = 0; u < DISP_U; ++u) {
+            if (i0 + 64 * u >= hi) break;  // wave-uniform
+            const int e = ids[u];
+            unsigned long long same = __ballot(e >= 0);
+            for (int b = 0; b < bits; ++b) {
+                const bool on = (e >> b) & 1;
+                const unsigned long long v = __ballot(on);
+                same &= on ? v : ~v;
+            }
+            if (e >= 0) {
+                const int at = cnt[wave * E + e], rank = __popcll(same & ((1ull << lane) - 1ull));
+                perm[at + rank] = (int)(i0 + 64 * u + lane);
+                if (rank == 0) cnt[wave * E + e] = at + __popcll(same);  // the wave's reads above come first: LDS works in order for a wave
+            }
         }
     }
 }
 
+__global__ __launch_bounds__(1024) void moe_dispatch_kernel(int64_t n, int E, int nw, const int* __restrict__ ids, int* __restrict__ offs, int* __restrict__ perm) {
+    extern __shared__ int lds[];
+    dispatch_lists(n, E, nw, [=](int64_t i) { return ids[i]; }, offs, perm, lds);
+}
+
 extern "C" int mi355_moe_dispatch(int64_t entries, int E, const int* ids, int* offs, int* perm, void* stream) {
     MI355_REQUIRE(entries > 0 && entries < (int64_t)1 << 31 && E > 0 && E <= 4096 && ids && offs && perm, "moe_dispatch: bad arguments");
-    moe_dispatch_kernel<<<1, 1024, sizeof(int) * (E + 1), ST(stream)>>>(entries, E, ids, offs, perm);
+    const int nw = disp_waves(E);
+    moe_dispatch_kernel<<<1, 1024, sizeof(int) * (nw * E + 16), ST(stream)>>>(entries, E, nw, ids, offs, perm);
     MI355_LAUNCH_CHECK("moe_dispatch");
+    return 0;
+}
+
+// The dispatch lists of EVERY layer of a step whose experts a table of the token ids picks: workgroup l takes layer l's table [vocab, top] at tables + meta[4 l]
+// (meta = {offset, top, E, 0}); its lists go to offs + l * (max_E + 1) and perm + l * tokens * max_top.
+__global__ __launch_bounds__(1024) void moe_table_dispatch_kernel(int64_t T, int vocab, int max_E, int max_top, int nw, const int* __restrict__ tok, const int* __restrict__ tables,
+                                                                  const int* __restrict__ meta, int* __restrict__ offs, int* __restrict__ perm) {
+    extern __shared__ int lds[];
+    const int l = blockIdx.x;
+    const int* table = tables + meta[4 * l];
+    const int top = min(meta[4 * l + 1], max_top), E = min(meta[4 * l + 2], max_E);
+    dispatch_lists(T * top, E, nw, [=](int64_t i) {
+        const unsigned t = (unsigned)i / (unsigned)top;
+        const int id = tok[t];
+        return (unsigned)id < (unsigned)vocab ? table[(int64_t)id * top + ((unsigned)i - t * top)] : -1;
+    }, offs + (int64_t)l * (max_E + 1), perm + (int64_t)l * T * max_top, lds);
+}
+
+extern "C" int mi355_moe_table_dispatch(int layers, int64_t tokens, int vocab, int max_E, int max_top, const int* tok, const int* tables, const int* meta, int* offs, int* perm,
+                                        void* stream) {
+    MI355_REQUIRE(layers > 0 && tokens > 0 && vocab > 0 && max_E > 0 && max_E <= 4096 && max_top > 0 && max_top <= max_E && tokens * max_top < (int64_t)1 << 31 && tok && tables && meta &&
+                      offs && perm, "moe_table_dispatch: bad arguments (experts <= 4096)");
+    const int nw = disp_waves(max_E);
+    moe_table_dispatch_kernel<<<layers, 1024, sizeof(int) * (nw * max_E + 16), ST(stream)>>>(tokens, vocab, max_E, max_top, nw, tok, tables, meta, offs, perm);
+    MI355_LAUNCH_CHECK("moe_table_dispatch");
     return 0;
 }

@@ -353,6 +353,8 @@ struct QkvRowsArgs {
     float* q_out;
     void* cache;
     int64_t lds_, ldq, ldc;
+    int unit_norm, tie_v;
+    float rot_amp;
     int src_dt, c_dt, H, G, GV, d, dv, dims, layout;  // H query heads and G key heads of d, GV value heads of dv
     float eps;
 };
@@ -366,7 +368,7 @@ __global__ __launch_bounds__(256) void qkv_rows_kernel(int64_t T, QkvRowsArgs p)
         const int hh = (int)(it % HT);
         const bool is_q = hh < p.H, is_k = !is_q && hh < p.H + p.G;
         const int n = (is_q || is_k) ? p.d : p.dv;
-        const int col0 = is_q ? hh * p.d : (is_k ? p.H * p.d + (hh - p.H) * p.d : (p.H + p.G) * p.d + (hh - p.H - p.G) * p.dv);
+        const int col0 = is_q ? hh * p.d : (is_k ? p.H * p.d + (hh - p.H) * p.d : (p.H + (p.tie_v ? 0 : p.G)) * p.d + (hh - p.H - p.G) * p.dv);
         const int64_t so = t * p.lds_ + col0;
         auto val = [&](int i) { return ldr_dt(p.src, p.src_dt, so + i) + (p.bias ? p.bias[col0 + i] : 0.f); };
         if (!is_q && !is_k) {
@@ -381,7 +383,7 @@ __global__ __launch_bounds__(256) void qkv_rows_kernel(int64_t T, QkvRowsArgs p)
         }
         const float* w = is_q ? p.qw : p.kw;
         float r = 1.0f;
-        if (w) {
+        if (w || p.unit_norm) {
             float s = 0.f;
             for (int i = lane; i < n; i += 64) {
                 const float a = val(i);
@@ -403,7 +405,7 @@ __global__ __launch_bounds__(256) void qkv_rows_kernel(int64_t T, QkvRowsArgs p)
             const int a = p.layout ? i : 2 * i, b = p.layout ? i + half : 2 * i + 1;
             const float u = val(a) * r * (w ? w[a] : 1.0f), v = val(b) * r * (w ? w[b] : 1.0f);
             const float ang = ps * p.freq[i];
-            const float c = cosf(ang), s = sinf(ang);
+            const float c = cosf(ang) * p.rot_amp, s = sinf(ang) * p.rot_amp;
             put(a, u * c - v * s);
             put(b, v * c + u * s);
         }
@@ -413,16 +415,19 @@ __global__ __launch_bounds__(256) void qkv_rows_kernel(int64_t T, QkvRowsArgs p)
 extern "C" int mi355_qkv_rows_append(int64_t tokens, int H, int G, int d, int dv, const void* src, int src_dt, int64_t ld_src, const float* bias, const float* qw,
                                      const float* kw, float eps, const float* qscale, int dims, int layout, const float* freq, const int* pos, const int* dst_row,
                                      float* q_out, int64_t ldq, void* cache, int c_dt, int64_t ldc, float qt_coef, int qt_every, const float* vmix, int64_t ldvm,
-                                     float lam, int v_heads, void* stream) {
+                                     float lam, int v_heads, int unit_norm, float rot_amp, int tie_v, void* stream) {
     const int GV = v_heads > 0 ? v_heads : G;
     MI355_REQUIRE(qt_every >= 0 && v_heads >= 0 && (!vmix || ldvm >= (int64_t)GV * dv), "qkv_rows_append: bad query temperature, value heads or value-mix rows");
     MI355_REQUIRE(tokens > 0 && H > 0 && G > 0 && d > 0 && dv > 0 && src && pos && dst_row && q_out && cache && rec_dt_ok(src_dt) && rec_dt_ok(c_dt), "qkv_rows_append: bad arguments");
     MI355_REQUIRE(dims >= 0 && dims % 2 == 0 && dims <= d && (dims == 0 || freq) && (layout == 0 || layout == 1), "qkv_rows_append: the rotated range must lie inside a head");
-    MI355_REQUIRE(ld_src >= (int64_t)(H + G) * d + (int64_t)GV * dv && ldq >= (int64_t)H * d && ldc >= (int64_t)G * d + (int64_t)GV * dv, "qkv_rows_append: rows too short");
+    MI355_REQUIRE(!tie_v || (GV == G && dv == d && !vmix), "qkv_rows_append: values that are the keys have the keys' heads and width, and are not mixed");
+    MI355_REQUIRE(!unit_norm || (!qw && !kw), "qkv_rows_append: a unit norm takes no weights");
+    MI355_REQUIRE(ld_src >= (int64_t)(H + G) * d + (tie_v ? 0 : (int64_t)GV * dv) && ldq >= (int64_t)H * d && ldc >= (int64_t)G * d + (int64_t)GV * dv, "qkv_rows_append: rows too short");
     QkvRowsArgs p;
     p.src = src, p.bias = bias, p.qw = qw, p.kw = kw, p.qscale = qscale, p.freq = freq, p.pos = pos, p.dst_row = dst_row, p.q_out = q_out, p.cache = cache;
     p.lds_ = ld_src, p.ldq = ldq, p.ldc = ldc, p.src_dt = src_dt, p.c_dt = c_dt, p.H = H, p.G = G, p.GV = GV, p.d = d, p.dv = dv, p.dims = dims, p.layout = layout, p.eps = eps;
     p.vmix = vmix, p.ldvm = ldvm, p.lam = lam, p.qt_coef = qt_coef, p.qt_every = qt_every;
+    p.unit_norm = unit_norm, p.rot_amp = rot_amp, p.tie_v = tie_v;
     qkv_rows_kernel<<<rec_rows_grid(tokens * (H + G + GV), 4), 256, 0, ST(stream)>>>(tokens, p);
     MI355_LAUNCH_CHECK("qkv_rows_append");
     return 0;

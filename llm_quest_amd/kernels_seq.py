@@ -3,7 +3,8 @@ post-sum LayerNorm on an fp32 residual stream, latent key/value rows, rotary emb
 gated linear attention and retention with carried state, the sigmoid and softmax routers and the grouped expert products (with gated epilogues), the residual
 sum with RMS norms in groups, short convolutions with carried inputs, query / key / value rows into a slot cache, the gated delta rule, gated activations,
 the residual sum between two norms (sandwich norms), pooled key / value rows, xIELU and sigmoid output gates on rows, the sum of parallel sublayers with a depth
-average, the join of differential attention (csrc/seqpar.hip, csrc/seqdep.hip).
+average, the join of differential attention (csrc/seqpar.hip, csrc/seqdep.hip), the mixing of several residual streams between two sublayers (csrc/seqhyp.hip),
+dispatch lists of experts that a table of the token ids picks.
 
 Activations are bf16 (serving mode: bf16 operands, fp32 accumulation) or fp32 (true 32-bit mode: every product is an fp32 FMA chain; the bf16
 weights are exactly representable and widened on load).  Whatever the mode, the residual stream, norm statistics, rotary angles, decays,
@@ -201,6 +202,22 @@ def moe_dispatch(ids, E):
     return offs, perm
 
 
+def moe_table_dispatch(tok, vocab, tables, meta, specs):
+    """The dispatch lists of every layer of a step whose experts a table of the token ids picks, in one launch.  ``tables`` int32: the layers' tables [vocab, top]
+    one after the other; ``specs`` = [(top, experts)] per layer, ``meta`` int32 [layers, 4] = (start of the table, top, experts, 0) on the device.  Returns per
+    layer (offs, perm) as ``moe_dispatch``."""
+    L.require_gpu(tok, tables, meta)
+    T, n = tok.numel(), len(specs)
+    _i32(tok, "moe_table_dispatch(tok)")
+    _i32(meta, "moe_table_dispatch(meta)", 4 * n)
+    _i32(tables, "moe_table_dispatch(tables)", sum(vocab * top for top, _ in specs))
+    max_top, max_e = max(t for t, _ in specs), max(e for _, e in specs)
+    offs = torch.empty((n, max_e + 1), dtype=I32, device=tok.device)
+    perm = torch.empty((n, T * max_top), dtype=I32, device=tok.device)
+    L.call("mi355_moe_table_dispatch", n, T, int(vocab), max_e, max_top, L.ptr(tok), L.ptr(tables), L.ptr(meta), L.ptr(offs), L.ptr(perm))
+    return [(offs[i, : e + 1], perm[i, : T * top]) for i, (top, e) in enumerate(specs)]
+
+
 def bgemm(a, b, c, M, N, Kd, batch=1, lda=None, a_bs=0, sbn=None, sbk=1, b_bs=0, ldc=None, c_bs=0, grp_offs=None, a_rows=None, a_div=1, c_rows=None,
           row_scale=None, epi=0, mfma=None, bias=None, limit=0.0, n_out=0):
     """The general strided product (see include/mi355_vlm.h).  Strides default to a's / c's row pitch and b stored [N, K]; the caller vouches that the
@@ -251,7 +268,7 @@ def attn_key_splits(n_seq, head_tiles, max_new, hm, max_keys, per_split=256):
 
 
 def latent_attn(q, k1, k2, v, out, H, hm, D1, D2, DV, q_hs, k1_hs, v_hs, o_hs, desc, max_new, scale, max_keys=0, kv_rep=1, window=0, keep_first=0, softcap=0.0,
-                sink=None, pool=0, pooled=None, pool_row0=None, chunk=0, sig_bias=None):
+                sink=None, pool=0, pooled=None, pool_row0=None, chunk=0, sig_bias=None, slope=None, gate=None):
     """Two-part-key causal attention over a ragged batch.  ``desc`` = (q_row0, n_new, past, k1_row0, k2_row0, v_row0) int32 [n_seq] each.  ``max_keys``
     (the longest sequence's keys, if the caller knows it) lets one-token steps over long caches spread a tile's keys over several workgroups.
     ``kv_rep``: query heads per key / value head (strides per key / value head).  ``window`` > 0: a query sees a key only ``window`` positions back, or
@@ -259,8 +276,14 @@ def latent_attn(q, k1, k2, v, out, H, hm, D1, D2, DV, q_hs, k1_hs, v_hs, o_hs, d
     denominator.  ``pool`` > 0: ``pooled`` = (pooled keys, pooled values), views laid out like ``k1`` / ``v`` with one mean row per ``pool`` tokens, first row
     of every sequence in ``pool_row0`` (int32 [n_seq]); a query sees the blocks that lie wholly before its window.  ``chunk`` > 0: positions are cut into chunks
     of that many from the sequence's first token on, and a query sees only the keys of its own chunk.  ``sig_bias`` (fp32 [H]): no softmax, a visible key's weight is
-    sigmoid(score + sig_bias[h]).  ``out`` has the dtype of the values, or fp32."""
-    L.require_gpu(q, k1, k2, v, out, sink, pool_row0, sig_bias, *desc)
+    sigmoid(score + sig_bias[h]).  ``slope`` (fp32 [H]): slope[h] * (i - j) is taken off the score of query position i and key j after scale and cap.  ``gate`` (fp32
+    [tokens, H * DV]): the output is multiplied element by element by its sigmoid.  ``out`` has the dtype of the values, or fp32."""
+    L.require_gpu(q, k1, k2, v, out, sink, pool_row0, sig_bias, slope, gate, *desc)
+    _vec32(slope, H, "latent_attn(slope)")
+    if gate is not None:
+        _rows(gate, "latent_attn(gate)")
+        if gate.dtype != F32 or tuple(gate.shape) != (q.shape[0], H * DV):
+            raise ValueError(f"latent_attn: the gate is fp32 [{q.shape[0]}, {H * DV}]")
     pk = pv = None
     if pool:
         pk, pv = pooled
@@ -282,17 +305,14 @@ def latent_attn(q, k1, k2, v, out, H, hm, D1, D2, DV, q_hs, k1_hs, v_hs, o_hs, d
         _i32(t, "latent_attn(desc)", n_seq)
     mfma = v.dtype == BF16
     splits, ws = 1, None
-    # A plain window leaves a tile window + its own tokens to see: that range is dealt out, in finer shares (a one-token step over it is a chain of
-    # dependent 64-key steps in very few workgroups).  A window that also keeps the first tokens is not dealt out: the kernel skips what lies between.
-    plain_window = window and window < max_keys and not keep_first
+    # A window or chunk leaves a tile a few keys to see (and the kept first tokens): those are dealt out, in finer shares (a one-token step over them is a chain of
+    # dependent 64-key steps in very few workgroups).
     reach = min(window or chunk, chunk or window)  # the most keys a row sees besides those of its own tile
-    if chunk and chunk < max_keys and not keep_first:
-        plain_window = True
-    if mfma and D1 + D2 <= 320 and DV <= 256 and max_keys and (not window or window >= max_keys or plain_window):
+    if mfma and D1 + D2 <= 320 and DV <= 256 and max_keys:
         head_tiles = -(-H // hm)
         tile_tokens = min(max_new, -(-128 // hm))
-        if plain_window:  # what a tile walks: its window, and one pooled row per block before it
-            rows = min(max_keys, reach + tile_tokens - 1) + (max(0, max_keys - window) // pool if pool else 0)
+        if reach and reach < max_keys:  # what a tile walks: kept tokens, its window, and one pooled row per block before it
+            rows = min(max_keys, keep_first + reach + tile_tokens - 1) + (max(0, max_keys - window) // pool if pool else 0)
             splits = attn_key_splits(n_seq, head_tiles, max_new, hm, rows, 128)
         else:
             splits = attn_key_splits(n_seq, head_tiles, max_new, hm, max_keys)
@@ -302,7 +322,8 @@ def latent_attn(q, k1, k2, v, out, H, hm, D1, D2, DV, q_hs, k1_hs, v_hs, o_hs, d
     L.call("mi355_latent_attn", n_seq, max_new, H, hm, D1, D2, DV, L.ptr(q), q.stride(0), q_hs, L.ptr(k1), k1.stride(0), k1_hs, L.ptr(k2), 0 if k2 is None else k2.stride(0),
            L.ptr(v), v.stride(0), v_hs, L.ptr(out), out.stride(0), o_hs, _dt(v), *[L.ptr(t) for t in desc], float(scale), 1 if mfma else 0, splits, L.ptr(ws),
            0 if ws is None else ws.numel(), int(kv_rep), int(window), int(keep_first), float(softcap or 0.0), L.ptr(sink), int(pool), L.ptr(pk), L.ptr(pv),
-           0 if pk is None else pk.stride(0), L.ptr(pool_row0), int(chunk), L.ptr(sig_bias), _dt(out))
+           0 if pk is None else pk.stride(0), L.ptr(pool_row0), int(chunk), L.ptr(sig_bias), _dt(out), L.ptr(slope), L.ptr(gate),
+           0 if gate is None else gate.stride(0))
     return out
 
 
@@ -363,10 +384,13 @@ def ragged_conv(x, w, state, row_seq, seq_off, slot, act=False, residual=False, 
     return y
 
 
-def qkv_rows_append(src, H, G, d, dv, bias, qw, kw, eps, qscale, dims, layout, freq, pos, dst_row, cache2d, q_temp=None, vmix=None, lam=0.0, v_heads=None):
+def qkv_rows_append(src, H, G, d, dv, bias, qw, kw, eps, qscale, dims, layout, freq, pos, dst_row, cache2d, q_temp=None, vmix=None, lam=0.0, v_heads=None, unit_norm=False,
+                    rot_amp=1.0, tie_v=False):
     """Rows [H x d | G x d | G x dv] -> fp32 queries [tokens, H * d] (bias, head norm, rotation, per-head scale) and key / value rows of ``cache2d``.
     ``q_temp`` = (coef, every): the query at position p is also multiplied by 1 + coef * ln(floor((p + 1) / every) + 1).  ``vmix`` (fp32 [tokens, G * dv],
-    any row pitch): the cached value is (1 - lam) v + lam * vmix.  ``v_heads``: that many value heads instead of G."""
+    any row pitch): the cached value is (1 - lam) v + lam * vmix.  ``v_heads``: that many value heads instead of G.  ``unit_norm``: query and key heads are divided by
+    their root mean square (no weight); ``rot_amp``: factor of cosine and sine; ``tie_v``: the rows are [H x d | G x d], the values are the keys as projected (bias
+    added, before norm and rotation)."""
     L.require_gpu(src, bias, qw, kw, qscale, freq, pos, dst_row, cache2d, vmix)
     GV = v_heads or G
     if vmix is not None:
@@ -379,9 +403,10 @@ def qkv_rows_append(src, H, G, d, dv, bias, qw, kw, eps, qscale, dims, layout, f
     _rows(src, "qkv_rows_append(src)")
     _rows(cache2d, "qkv_rows_append(cache)")
     T = src.shape[0]
-    if src.shape[1] != (H + G) * d + GV * dv or cache2d.shape[1] != G * d + GV * dv:
+    n_in = (H + G) * d + (0 if tie_v else GV * dv)
+    if src.shape[1] != n_in or cache2d.shape[1] != G * d + GV * dv:
         raise ValueError("qkv_rows_append: row widths do not match the head layout")
-    for t, n in ((bias, (H + G) * d + GV * dv), (qw, d), (kw, d), (qscale, H), (freq, dims // 2)):
+    for t, n in ((bias, n_in), (qw, d), (kw, d), (qscale, H), (freq, dims // 2)):
         if t is not None and (t.dtype != F32 or not t.is_contiguous() or t.numel() < n):
             raise ValueError("qkv_rows_append: vectors are contiguous fp32 of the layout's sizes")
     _i32(pos, "qkv_rows_append(pos)", T)
@@ -389,7 +414,7 @@ def qkv_rows_append(src, H, G, d, dv, bias, qw, kw, eps, qscale, dims, layout, f
     q = torch.empty((T, H * d), dtype=F32, device=src.device)
     L.call("mi355_qkv_rows_append", T, H, G, d, dv, L.ptr(src), _dt(src), src.stride(0), L.ptr(bias), L.ptr(qw), L.ptr(kw), float(eps), L.ptr(qscale), int(dims), int(layout),
            L.ptr(freq), L.ptr(pos), L.ptr(dst_row), L.ptr(q), q.stride(0), L.ptr(cache2d), _dt(cache2d), cache2d.stride(0), coef, every, L.ptr(vmix),
-           0 if vmix is None else vmix.stride(0), float(lam), int(GV))
+           0 if vmix is None else vmix.stride(0), float(lam), int(GV), 1 if unit_norm else 0, float(rot_amp), 1 if tie_v else 0)
     return q
 
 
@@ -773,3 +798,49 @@ def scaled_rope_frequencies(dims, base, scaling, device):
         mid = (1.0 - smooth) * f / fac + smooth * f
         f = torch.where(wl < orig / hi, f, torch.where(wl > orig / lo, f / fac, mid))
     return f.to(F32).to(device)
+
+
+def yarn_rope_frequencies(dims, base, scaling, device):
+    """(fp32 [dims / 2], amplitude): rotary frequencies for a longer context than the one trained on.  With d(t) = dims ln(original / (2 pi t)) / (2 ln base) the
+    entry whose wavelength makes t turns over the original context, frequencies below entry floor(d(fast)) stay, those from ceil(d(slow)) on are divided by
+    ``factor``, between the two a linear ramp over the entry blends them; cosine and sine are multiplied by 0.1 ln(factor) + 1.  Evaluated in double."""
+    import math
+
+    fac, orig = float(scaling["factor"]), float(scaling["original"])
+    i = torch.arange(dims // 2, dtype=torch.float64)
+    f = torch.pow(torch.tensor(float(base), dtype=torch.float64), -2.0 * i / dims)
+    entry = lambda turns: dims * math.log(orig / (2.0 * math.pi * float(turns))) / (2.0 * math.log(float(base)))
+    lo, hi = max(math.floor(entry(scaling["fast"])), 0), min(math.ceil(entry(scaling["slow"])), dims - 1)
+    ramp = ((i - lo) / max(hi - lo, 0.001)).clamp(0.0, 1.0)
+    return (f / fac * ramp + f * (1.0 - ramp)).to(F32).to(device), 0.1 * math.log(fac) + 1.0
+
+
+def hyper_mix(x, S, y=None, parts=1, y_scale=1.0, mix=None, put=None, read=None, rows=None, x_out=None, want_u=False, norm=None, eps=0.0, out_dtype=None):
+    """What lies between two sublayers of a decoder with ``S`` residual streams.  ``x`` fp32 [tokens, S, width], or [tokens, width]: all streams alike.  With a
+    pending sublayer output ``y`` ([tokens * parts, width], bf16 or fp32) every stream becomes sum_s mix[s, t] x_s + put[t] * y_scale * (sum of y's parts), all from
+    the old streams (``mix`` fp32 [S, S] = [from, to], ``put`` fp32 [S]); ``x_out`` (True: a new tensor, or a tensor, or None) receives them.  ``read`` (fp32 [S]):
+    u = sum_s read[s] x_s; ``norm`` (fp32 [width]): its RMS norm times that weight is returned in ``out_dtype``.  ``rows`` (int64): only these tokens.
+    Returns (x_out or None, normed or None, u or None)."""
+    L.require_gpu(x, y, mix, put, read, rows, norm, x_out if torch.is_tensor(x_out) else None)
+    n_tok, width = x.shape[0], x.shape[-1]
+    if x.dtype != F32 or x.stride(-1) != 1 or (x.dim() == 3 and x.shape[1] != S) or x.dim() not in (2, 3):
+        raise ValueError("hyper_mix: x is fp32 [tokens, S, width], or [tokens, width]")
+    T = n_tok if rows is None else rows.numel()
+    if rows is not None and (rows.dtype != torch.int64 or not rows.is_contiguous()):
+        raise ValueError("hyper_mix: rows are contiguous int64")
+    if y is not None:
+        _rows(y, "hyper_mix(y)")
+        if tuple(y.shape) != (n_tok * parts, width) or mix is None or put is None:
+            raise ValueError(f"hyper_mix: the sublayer output is [{n_tok * parts}, {width}] and comes with mix and put")
+    for v, n, name in ((mix, S * S, "mix"), (put, S, "put"), (read, S, "read"), (norm, width, "norm")):
+        if v is not None and (v.dtype != F32 or not v.is_contiguous() or v.numel() != n):
+            raise ValueError(f"hyper_mix({name}): contiguous fp32 of {n} entries required")
+    if x_out is True:
+        x_out = torch.empty((T, S, width), dtype=F32, device=x.device)
+    elif x_out is not None and (x_out.dtype != F32 or not x_out.is_contiguous() or tuple(x_out.shape) != (T, S, width)):
+        raise ValueError("hyper_mix: x_out is contiguous fp32 [tokens, S, width]")
+    out = torch.empty((T, width), dtype=out_dtype or F32, device=x.device) if norm is not None else None
+    u = torch.empty((T, width), dtype=F32, device=x.device) if want_u else None
+    L.call("mi355_hyper_mix", T, width, S, L.ptr(x), x.stride(0), x.stride(1) if x.dim() == 3 else 0, L.ptr(y), 0 if y is None else _dt(y), 0 if y is None else y.stride(0), int(parts),
+           float(y_scale), L.ptr(mix), L.ptr(put), L.ptr(read), L.ptr(rows), L.ptr(x_out), L.ptr(u), L.ptr(norm), float(eps), L.ptr(out), 0 if out is None else _dt(out))
+    return x_out, out, u

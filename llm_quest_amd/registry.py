@@ -52,11 +52,18 @@ def _foderax(model_dir, act_dtype, device):
     return load_foderax(model_dir, act_dtype, device)
 
 
+def _pavisun(model_dir, act_dtype, device):
+    from llm_quest_amd.pavisun.pavisun_weight_loading import load_pavisun
+
+    return load_pavisun(model_dir, act_dtype, device)
+
+
 register("Gemepel", _gemepel)
 register("Mepatar", _mepatar)
 register("Mopalorn", _mopalorn)
 register("Gepilix", _gepilix)
 register("Foderax", _foderax)
+register("Pavisun", _pavisun)
 
 
 def load_model(model_dir, dtype="bfloat16", device="cuda"):
