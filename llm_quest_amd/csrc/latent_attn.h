@@ -1,4 +1,4 @@
-// Arguments of the ragged-batch attention kernels (latent_attn.hip: every option; latent_attn_full.hip: every key j <= i).
+// Arguments of the ragged-batch attention kernels (latent_attn.hip: every option; latent_attn_full.hip, latent_attn_win.hip: the lean MFMA kernel).
 #pragma once
 #include "common.h"
 
@@ -57,3 +57,5 @@ __device__ __forceinline__ float gate_of(float g) { return 1.0f / (1.0f + expf(-
 // Launches the kernel for attention over every key j <= i (no window, chunk, pooled rows or cap; scale > 0; rows 16-byte aligned, widths multiples of 8) if it
 // holds these sizes; false: the caller takes the general kernel.  Partial results under key splits have the general kernel's layout.
 bool latent_attn_full_launch(const LatAttnArgs& p, dim3 grid, hipStream_t st);
+// The same under a window or chunk, with capped scores or a distance bias (no pooled rows, no sigmoid weights).
+bool latent_attn_win_launch(const LatAttnArgs& p, dim3 grid, hipStream_t st);

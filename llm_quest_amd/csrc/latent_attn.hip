@@ -16,7 +16,7 @@
 // keys and values) against 64 keys at a time.
 //
 // Three compute paths: fp32 FMA through LDS (any operand type: the true-fp32 mode), bf16 MFMA (v_mfma_f32_32x32x8_bf16_1k) for bf16 keys / values with every
-// option, and -- latent_attn_full.hip -- a leaner bf16 MFMA kernel for the cases that see every key j <= i without a cap.
+// option, and -- latent_attn_full.h -- a leaner bf16 MFMA kernel for aligned rows without pooled blocks (sigmoid weights: only where every key j <= i is seen).
 #include "latent_attn.h"
 
 #define ST(s) ((hipStream_t)(s))
@@ -577,9 +577,10 @@ extern "C" int mi355_latent_attn(int n_seq, int max_new, int H, int hm, int D1, 
         const int vec_ok = D1 % 8 == 0 && D2 % 8 == 0 && DV % 8 == 0 && ldk1 % 8 == 0 && ldk2 % 8 == 0 && ldv % 8 == 0 && k1_hs % 8 == 0 && v_hs % 8 == 0 &&
                            ((uintptr_t)K1 & 15) == 0 && ((uintptr_t)K2 & 15) == 0 && ((uintptr_t)V & 15) == 0 &&
                            (pool == 0 || (ldp % 8 == 0 && ((uintptr_t)PK & 15) == 0 && ((uintptr_t)PV & 15) == 0));
-        const bool o_vec = ldo % 4 == 0 && o_hs % 4 == 0 && ((uintptr_t)O & 15) == 0;
-        if (window == 0 && chunk == 0 && pool == 0 && softcap == 0.f && !slope && !gate && scale > 0.f && vec_ok && o_vec && latent_attn_full_launch(p, grid, ST(stream))) {
-            // every key j <= i, aligned rows: done
+        const bool o_vec = ldo % 4 == 0 && o_hs % 4 == 0 && ((uintptr_t)O & 15) == 0 && (!gate || (ldg % 4 == 0 && ((uintptr_t)gate & 15) == 0));
+        const bool lean = pool == 0 && scale > 0.f && vec_ok && o_vec, all_keys = window == 0 && chunk == 0 && softcap == 0.f && !slope;
+        if (lean && (all_keys ? latent_attn_full_launch(p, grid, ST(stream)) : latent_attn_win_launch(p, grid, ST(stream)))) {
+            // aligned rows, sizes the lean kernel holds: done
         } else if (sig_bias) launch_mfma_dk<true>(p, grid, vec_ok, ST(stream));
         else launch_mfma_dk<false>(p, grid, vec_ok, ST(stream));
         MI355_LAUNCH_CHECK("latent_attn(mfma)");
