@@ -12,9 +12,10 @@
 // weights kept in bf16 -- exactly representable -- and widened on load, fp32 FMA accumulation in a fixed k order, so a row's result does not depend
 // on which other rows share its tile).
 //
-// Two compute paths:
+// Compute paths:
 //   * FMA: 64 x 64 tile, 256 threads, 4 x 4 outputs per thread, k in steps of 16 through LDS (any operand type);
-//   * MFMA (bf16 A and B): the same tile, four waves of 32 x 32 on v_mfma_f32_32x32x8_bf16_1k, k in steps of 32.
+//   * MFMA (bf16 A and B): the same tile, four waves of 32 x 32 on v_mfma_f32_32x32x8_bf16_1k, k in steps of 32; a 128 x 128 tile on v_mfma_f32_32x32x16_bf16 for
+//     weights stored [out, in]; and, for few rows in all groups together, a stream of the weights that deals k to the waves of a workgroup.
 #include "common.h"
 
 #define ST(s) ((hipStream_t)(s))
@@ -230,12 +231,16 @@ __global__ __launch_bounds__(256) void bgemm_mfma_kernel(BgemmArgs p) {
         }
 }
 
-// ---- MFMA path, 128 x 128 tile: four waves of 64 x 64 (2 x 2 blocks of 32 x 32), k in steps of 32; the next step's operands are fetched into registers
-// while the current step multiplies from LDS (one LDS stage, two barriers per step).  Four LDS fragment reads feed four MFMAs.
+// ---- MFMA path, 128 x 128 tile: four waves of 64 x 64 (2 x 2 blocks of v_mfma_f32_32x32x16_bf16: lane l supplies A[m = l % 32][k = 8 * (l / 32) .. +8] and B[n = l % 32]
+// [same k]), k in steps of 64; the next step's operands are fetched into registers while the current step multiplies from LDS (one LDS stage, two barriers per step).
+// Four LDS fragment reads feed four MFMAs.
 #define TM 128
+#define TK 64
+// VEC: both operands in 16-byte words (K and every stride a multiple of 8, B stored [out, in]).
+template <bool VEC>
 __global__ __launch_bounds__(256) void bgemm_mfma128_kernel(BgemmArgs p) {
-    __shared__ __attribute__((aligned(16))) bf16_t As[TM][MK + MPAD];
-    __shared__ __attribute__((aligned(16))) bf16_t Bs[TM][MK + MPAD];
+    __shared__ __attribute__((aligned(16))) bf16_t As[TM][TK + MPAD];
+    __shared__ __attribute__((aligned(16))) bf16_t Bs[TM][TK + MPAD];
     const int b = blockIdx.z;
     int row0 = 0, rows = p.M;
     if (p.grp_offs) {
@@ -251,41 +256,43 @@ __global__ __launch_bounds__(256) void bgemm_mfma128_kernel(BgemmArgs p) {
     const int64_t b_base = (int64_t)b * p.b_bs;
     const bool a_vec = (p.lda % 8 == 0) && (p.a_bs % 8 == 0) && (((uintptr_t)p.A & 15) == 0);
     const bool b_vec = b_kfast && (p.sbn % 8 == 0) && (p.b_bs % 8 == 0) && (((uintptr_t)p.B & 15) == 0);
-    // loader roles: chunk c = tid + 256 i (i < 2): row c / 4, k offset (c % 4) * 8
-    int64_t a_base[2];
-    int lr[2], lk[2];
+    // loader roles: chunk c = tid + 256 i (i < 4): row c / 8, k offset (c % 8) * 8
+    int64_t a_base[4];
+    const int lr0 = tid >> 3, lk = (tid & 7) * 8;
 #pragma unroll
-    for (int i = 0; i < 2; ++i) {
-        const int c = tid + 256 * i;
-        lr[i] = c >> 2, lk[i] = (c & 3) * 8;
+    for (int i = 0; i < 4; ++i) {
         a_base[i] = -1;
-        if (m0 + lr[i] < rows) {
-            const int r = row0 + m0 + lr[i];
+        if (m0 + lr0 + 32 * i < rows) {
+            const int r = row0 + m0 + lr0 + 32 * i;
             const int64_t arow = p.a_rows ? p.a_rows[r] / p.a_div : r;
             a_base[i] = (int64_t)b * p.a_bs + arow * p.lda;
         }
     }
-    u32x4 ra[2], rb[2];
+    u32x4 ra[4], rb[4];
     auto fetch = [&](int k0) {
 #pragma unroll
-        for (int i = 0; i < 2; ++i) {
+        for (int i = 0; i < 4; ++i) {
             u32x4 va = {0u, 0u, 0u, 0u}, vb = {0u, 0u, 0u, 0u};
             if (a_base[i] >= 0) {
-                if (a_vec && k0 + lk[i] + 8 <= p.K) va = *(const u32x4*)(A + a_base[i] + k0 + lk[i]);
+                if (VEC) {
+                    if (k0 + lk < p.K) va = *(const u32x4*)(A + a_base[i] + k0 + lk);
+                } else if (a_vec && k0 + lk + 8 <= p.K) va = *(const u32x4*)(A + a_base[i] + k0 + lk);
                 else {
                     bf16_t e[8];
 #pragma unroll
-                    for (int j = 0; j < 8; ++j) e[j] = k0 + lk[i] + j < p.K ? A[a_base[i] + k0 + lk[i] + j] : (bf16_t)0;
+                    for (int j = 0; j < 8; ++j) e[j] = k0 + lk + j < p.K ? A[a_base[i] + k0 + lk + j] : (bf16_t)0;
                     va = u32x4{(unsigned)e[0] | ((unsigned)e[1] << 16), (unsigned)e[2] | ((unsigned)e[3] << 16), (unsigned)e[4] | ((unsigned)e[5] << 16), (unsigned)e[6] | ((unsigned)e[7] << 16)};
                 }
             }
-            const int n = n0 + lr[i];
+            const int n = n0 + lr0 + 32 * i;
             if (n < p.N) {
-                if (b_vec && k0 + lk[i] + 8 <= p.K) vb = *(const u32x4*)(B + b_base + (int64_t)n * p.sbn + k0 + lk[i]);
+                if (VEC) {
+                    if (k0 + lk < p.K) vb = *(const u32x4*)(B + b_base + (int64_t)n * p.sbn + k0 + lk);
+                } else if (b_vec && k0 + lk + 8 <= p.K) vb = *(const u32x4*)(B + b_base + (int64_t)n * p.sbn + k0 + lk);
                 else {
                     bf16_t e[8];
 #pragma unroll
-                    for (int j = 0; j < 8; ++j) e[j] = k0 + lk[i] + j < p.K ? B[b_base + (int64_t)n * p.sbn + (int64_t)(k0 + lk[i] + j) * p.sbk] : (bf16_t)0;
+                    for (int j = 0; j < 8; ++j) e[j] = k0 + lk + j < p.K ? B[b_base + (int64_t)n * p.sbn + (int64_t)(k0 + lk + j) * p.sbk] : (bf16_t)0;
                     vb = u32x4{(unsigned)e[0] | ((unsigned)e[1] << 16), (unsigned)e[2] | ((unsigned)e[3] << 16), (unsigned)e[4] | ((unsigned)e[5] << 16), (unsigned)e[6] | ((unsigned)e[7] << 16)};
                 }
             }
@@ -301,23 +308,23 @@ __global__ __launch_bounds__(256) void bgemm_mfma128_kernel(BgemmArgs p) {
             for (int e = 0; e < 16; ++e) acc[i][j][e] = 0.f;
     const int wm = (wave >> 1) * 64, wn = (wave & 1) * 64;
     fetch(0);
-    for (int k0 = 0; k0 < p.K; k0 += MK) {
+    for (int k0 = 0; k0 < p.K; k0 += TK) {
         __syncthreads();  // the previous step's fragments are read
 #pragma unroll
-        for (int i = 0; i < 2; ++i) {
-            *(u32x4*)&As[lr[i]][lk[i]] = ra[i];
-            *(u32x4*)&Bs[lr[i]][lk[i]] = rb[i];
+        for (int i = 0; i < 4; ++i) {
+            *(u32x4*)&As[lr0 + 32 * i][lk] = ra[i];
+            *(u32x4*)&Bs[lr0 + 32 * i][lk] = rb[i];
         }
         __syncthreads();
-        if (k0 + MK < p.K) fetch(k0 + MK);
+        if (k0 + TK < p.K) fetch(k0 + TK);
 #pragma unroll
-        for (int kk = 0; kk < MK; kk += 8) {
-            const bf16x4 a0 = *(const bf16x4*)&As[wm + ln][kk + 4 * hf], a1 = *(const bf16x4*)&As[wm + 32 + ln][kk + 4 * hf];
-            const bf16x4 b0 = *(const bf16x4*)&Bs[wn + ln][kk + 4 * hf], b1 = *(const bf16x4*)&Bs[wn + 32 + ln][kk + 4 * hf];
-            acc[0][0] = __builtin_amdgcn_mfma_f32_32x32x8bf16_1k(a0, b0, acc[0][0], 0, 0, 0);
-            acc[0][1] = __builtin_amdgcn_mfma_f32_32x32x8bf16_1k(a0, b1, acc[0][1], 0, 0, 0);
-            acc[1][0] = __builtin_amdgcn_mfma_f32_32x32x8bf16_1k(a1, b0, acc[1][0], 0, 0, 0);
-            acc[1][1] = __builtin_amdgcn_mfma_f32_32x32x8bf16_1k(a1, b1, acc[1][1], 0, 0, 0);
+        for (int kk = 0; kk < TK; kk += 16) {
+            const bf16x8 a0 = *(const bf16x8*)&As[wm + ln][kk + 8 * hf], a1 = *(const bf16x8*)&As[wm + 32 + ln][kk + 8 * hf];
+            const bf16x8 b0 = *(const bf16x8*)&Bs[wn + ln][kk + 8 * hf], b1 = *(const bf16x8*)&Bs[wn + 32 + ln][kk + 8 * hf];
+            acc[0][0] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a0, b0, acc[0][0], 0, 0, 0);
+            acc[0][1] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a0, b1, acc[0][1], 0, 0, 0);
+            acc[1][0] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a1, b0, acc[1][0], 0, 0, 0);
+            acc[1][1] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a1, b1, acc[1][1], 0, 0, 0);
         }
     }
 #pragma unroll
@@ -354,6 +361,94 @@ __global__ __launch_bounds__(256) void bgemm_mfma128_kernel(BgemmArgs p) {
             }
 }
 
+// ---- MFMA path for few rows per group (one-token steps through a mixture's experts): bound by the stream of the weights.  A workgroup is eight waves on 32 rows x 32
+// columns (GLU: the 32 gate and the 32 up columns of one block); the waves deal the k range among themselves, read both operands straight from memory in
+// fragment form -- 16 bytes per lane, SU steps of 16 in flight while the previous SU multiply -- and their partial sums meet in LDS.
+#define SW 8
+#define SU 4
+#define STREAM_ROWS 256  // up to this many sorted rows in all groups together
+template <bool GLU>
+__global__ __launch_bounds__(64 * SW) void bgemm_stream_kernel(BgemmArgs p) {
+    constexpr int NB = GLU ? 2 : 1;
+    __shared__ float red[SW][NB][16][64];
+    const int b = blockIdx.z, row0 = p.grp_offs[b], rows = p.grp_offs[b + 1] - row0;
+    const int m0 = blockIdx.y * 32, n0 = blockIdx.x * 32 * NB;
+    if (m0 >= rows) return;
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, ln = lane & 31, hf = lane >> 5;
+    const bf16_t* a_row = nullptr;
+    if (m0 + ln < rows) {
+        const int r = row0 + m0 + ln;
+        a_row = (const bf16_t*)p.A + (int64_t)b * p.a_bs + (int64_t)(p.a_rows ? p.a_rows[r] / p.a_div : r) * p.lda;
+    }
+    const bf16_t* b_row[NB];
+#pragma unroll
+    for (int j = 0; j < NB; ++j) b_row[j] = n0 + 32 * j + ln < p.N ? (const bf16_t*)p.B + (int64_t)b * p.b_bs + (int64_t)(n0 + 32 * j + ln) * p.sbn : nullptr;
+    const int steps = (p.K + 15) / 16, per = (steps + SW - 1) / SW, s0 = min(wave * per, steps), s1 = min(s0 + per, steps);
+    const u32x4 zero = {0u, 0u, 0u, 0u};
+    u32x4 fa[SU], fb[SU][NB];
+    auto fetch = [&](int st) {
+#pragma unroll
+        for (int u = 0; u < SU; ++u) {
+            const int k = (st + u) * 16 + 8 * hf;  // K is a multiple of 8
+            const bool in = st + u < s1 && k < p.K;
+            fa[u] = in && a_row ? *(const u32x4*)(a_row + k) : zero;
+#pragma unroll
+            for (int j = 0; j < NB; ++j) fb[u][j] = in && b_row[j] ? *(const u32x4*)(b_row[j] + k) : zero;
+        }
+    };
+    f32x16 acc[NB];
+#pragma unroll
+    for (int j = 0; j < NB; ++j)
+#pragma unroll
+        for (int e = 0; e < 16; ++e) acc[j][e] = 0.f;
+    fetch(s0);
+    for (int st = s0; st < s1; st += SU) {
+        u32x4 ca[SU], cb[SU][NB];
+#pragma unroll
+        for (int u = 0; u < SU; ++u) {
+            ca[u] = fa[u];
+#pragma unroll
+            for (int j = 0; j < NB; ++j) cb[u][j] = fb[u][j];
+        }
+        if (st + SU < s1) fetch(st + SU);
+#pragma unroll
+        for (int u = 0; u < SU; ++u)
+#pragma unroll
+            for (int j = 0; j < NB; ++j) acc[j] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8, ca[u]), __builtin_bit_cast(bf16x8, cb[u][j]), acc[j], 0, 0, 0);
+    }
+#pragma unroll
+    for (int j = 0; j < NB; ++j)
+#pragma unroll
+        for (int e = 0; e < 16; ++e) red[wave][j][e][lane] = acc[j][e];
+    __syncthreads();
+    const int n = n0 / NB + ln;
+#pragma unroll
+    for (int q = 0; q < 16 / SW; ++q) {
+        const int e = wave * (16 / SW) + q, m = m0 + 8 * (e >> 2) + 4 * hf + (e & 3);
+        float v[NB];
+#pragma unroll
+        for (int j = 0; j < NB; ++j) {
+            v[j] = 0.f;
+#pragma unroll
+            for (int w = 0; w < SW; ++w) v[j] += red[w][j][e][lane];
+        }
+        if (m >= rows || n >= (GLU ? p.n_out : p.N)) continue;
+        const int r = row0 + m;
+        const int64_t crow = p.c_rows ? p.c_rows[r] : r;
+        float x;
+        if constexpr (GLU) {
+            x = gated_act(p.epi, v[0], v[NB - 1], p.limit);
+        } else {
+            x = v[0] + (p.bias ? p.bias[n] : 0.f);
+            if (p.epi == 1) x = x > 0.f ? x * x : 0.f;
+        }
+        x *= p.row_scale ? p.row_scale[crow] : 1.0f;
+        const int64_t ci = (int64_t)b * p.c_bs + crow * p.ldc + n;
+        if (p.c_dt == MI355_DT_F32) ((float*)p.C)[ci] = x;
+        else ((bf16_t*)p.C)[ci] = f2bf(x);
+    }
+}
+
 extern "C" int mi355_bgemm(int batch, int M, int N, int K, const void* A, int a_dt, int64_t lda, int64_t a_bs, const void* B, int b_dt, int64_t sbn, int64_t sbk,
                            int64_t b_bs, void* C, int c_dt, int64_t ldc, int64_t c_bs, const int* grp_offs, const int* a_rows, int a_div, const int* c_rows,
                            const float* row_scale, int epi, int use_mfma, const float* bias, float limit, int n_out, void* stream) {
@@ -373,10 +468,20 @@ extern "C" int mi355_bgemm(int batch, int M, int N, int K, const void* A, int a_
     p.bias = bias;
     p.limit = limit, p.n_out = n_out;
     p.epi = epi, p.a_dt = a_dt, p.b_dt = b_dt, p.c_dt = c_dt;
+    const bool vec = sbk == 1 && K % 8 == 0 && lda % 8 == 0 && a_bs % 8 == 0 && sbn % 8 == 0 && b_bs % 8 == 0 && ((uintptr_t)A & 15) == 0 && ((uintptr_t)B & 15) == 0;
+    if (use_mfma && grp_offs && M <= STREAM_ROWS && K >= 256 && vec) {
+        const dim3 grid((N + (epi >= 2 ? 63 : 31)) / (epi >= 2 ? 64 : 32), (M + 31) / 32, batch);
+        if (epi >= 2) bgemm_stream_kernel<true><<<grid, 64 * SW, 0, ST(stream)>>>(p);
+        else bgemm_stream_kernel<false><<<grid, 64 * SW, 0, ST(stream)>>>(p);
+        MI355_LAUNCH_CHECK("bgemm(stream)");
+        return 0;
+    }
     if (use_mfma && ((sbk == 1 && N >= 128 && K >= 64) || epi >= 2)) {  // (a gated epilogue needs a gate and its up in one lane: this kernel's 64 columns per wave)  // the large tile: weights stored [out, in], enough columns to fill it
         const int64_t my128 = ((int64_t)M + TM - 1) / TM;
         MI355_REQUIRE(my128 <= 65535, "bgemm: too many row tiles");
-        bgemm_mfma128_kernel<<<dim3((N + TM - 1) / TM, (unsigned)my128, batch), 256, 0, ST(stream)>>>(p);
+        const dim3 grid((N + TM - 1) / TM, (unsigned)my128, batch);
+        if (vec) bgemm_mfma128_kernel<true><<<grid, 256, 0, ST(stream)>>>(p);
+        else bgemm_mfma128_kernel<false><<<grid, 256, 0, ST(stream)>>>(p);
         MI355_LAUNCH_CHECK("bgemm");
         return 0;
     }

@@ -34,11 +34,14 @@ static inline bool dt_ok(int dt) { return dt == MI355_DT_BF16 || dt == MI355_DT_
 
 // ------------------------------------------------------------------------------------------- embedding + hashed bigram
 // out[t] = table[tok[t]] * scale + bigram[row(t)],  row = (prev * mul_prev + tok * mul_cur) mod buckets, or `buckets` when prev < 0
+// WPR waves share a row: 4 in steps of few rows (a row's loads are all in flight at once), 1 in prompts.
+template <int WPR>
 __global__ __launch_bounds__(256) void embed_hash_kernel(int64_t T, int width, int vocab, const int* __restrict__ tok, const int* __restrict__ prev,
                                                          const bf16_t* __restrict__ table, float scale, const bf16_t* __restrict__ bigram, int buckets,
                                                          int mul_prev, int mul_cur, float* __restrict__ out) {
-    const int lane = threadIdx.x & 63;
-    for (int64_t t = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6); t < T; t += (int64_t)gridDim.x * 4) {
+    constexpr int ROWS = 4 / WPR;
+    const int i0 = WPR == 1 ? threadIdx.x & 63 : threadIdx.x;
+    for (int64_t t = (int64_t)blockIdx.x * ROWS + (WPR == 1 ? threadIdx.x >> 6 : 0); t < T; t += (int64_t)gridDim.x * ROWS) {
         const int id = tok[t];
         const bool ok = id >= 0 && id < vocab;
         const bf16_t* e = table + (int64_t)(ok ? id : 0) * width;
@@ -50,7 +53,8 @@ __global__ __launch_bounds__(256) void embed_hash_kernel(int64_t T, int width, i
             if (row < 0) row += buckets;
             b = bigram + row * width;
         }
-        for (int i = lane; i < width; i += 64) {
+#pragma unroll 8
+        for (int i = i0; i < width; i += 64 * WPR) {
             float v = ok ? bf2f(e[i]) * scale : 0.f;
             if (b) v += bf2f(b[i]);
             out[t * width + i] = v;
@@ -62,8 +66,10 @@ extern "C" int mi355_embed_hash_fwd(int64_t tokens, int width, int vocab, const 
                                     const void* bigram, int buckets, int mul_prev, int mul_cur, float* out, void* stream) {
     MI355_REQUIRE(tokens > 0 && width > 0 && vocab > 0 && tok && table && out, "embed_hash_fwd: bad arguments");
     MI355_REQUIRE(!bigram || (prev && buckets > 0), "embed_hash_fwd: a bigram table needs the previous tokens and a bucket count");
-    embed_hash_kernel<<<rows_grid(tokens, 4), 256, 0, ST(stream)>>>(tokens, width, vocab, tok, prev, (const bf16_t*)table, scale, (const bf16_t*)bigram,
-                                                                    buckets, mul_prev, mul_cur, out);
+    const bool few = tokens < 1024;
+    auto* kernel = few ? &embed_hash_kernel<4> : &embed_hash_kernel<1>;
+    kernel<<<rows_grid(tokens, few ? 1 : 4), 256, 0, ST(stream)>>>(tokens, width, vocab, tok, prev, (const bf16_t*)table, scale, (const bf16_t*)bigram, buckets, mul_prev, mul_cur,
+                                                                   out);
     MI355_LAUNCH_CHECK("embed_hash_fwd");
     return 0;
 }

@@ -412,6 +412,105 @@ __global__ __launch_bounds__(256) void qkv_rows_kernel(int64_t T, QkvRowsArgs p)
     }
 }
 
+// The same on rows of 16-byte words (widths multiples of 4, the rotated range of 8 in layout 1).  LPH lanes (a power of two) share a head, 64 / LPH heads a wave at a time;
+// a lane owns one unit of every head it meets -- layout 1: entries 4 u .. + 3 and the four they turn with, or four entries that pass; layout 0: four entries -- so
+// cosine and sine of its angles are taken once per token.  A token's heads are dealt to `chunks` waves (steps of few rows) or stay with one.
+template <int LAYOUT>
+__global__ __launch_bounds__(256) void qkv_rows_vec_kernel(int64_t T, QkvRowsArgs p, int LPH, int chunks) {
+    const int lane = threadIdx.x & 63, u = lane & (LPH - 1), hw = lane / LPH, HPW = 64 / LPH;
+    const int HK = p.H + p.G, HT = HK + (p.tie_v ? 0 : p.GV);
+    const int half = p.dims / 2;
+    const bool turns = LAYOUT ? 4 * u < half : 4 * u < p.dims;
+    const int a0 = LAYOUT && !turns ? p.dims + 4 * u - half : 4 * u, a1 = a0 + half;  // the unit's entries; a1: their partners in layout 1
+    const bool mine = a0 < p.d;
+    for (int64_t it = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6); it < T * chunks; it += (int64_t)gridDim.x * 4) {
+        const int64_t t = it / chunks;
+        const int pos = p.pos[t];
+        const int64_t row = (int64_t)p.dst_row[t] * p.ldc;
+        const float qt = p.qt_every > 0 ? 1.0f + p.qt_coef * logf((float)((pos + 1) / p.qt_every + 1)) : 1.0f;
+        float c[4] = {1.f, 1.f, 1.f, 1.f}, s[4] = {0.f, 0.f, 0.f, 0.f};
+        if (turns && mine) {
+#pragma unroll
+            for (int e = 0; e < (LAYOUT ? 4 : 2); ++e) {
+                const float ang = (float)pos * p.freq[LAYOUT ? 4 * u + e : 2 * u + e];
+                c[e] = cosf(ang) * p.rot_amp, s[e] = sinf(ang) * p.rot_amp;
+            }
+        }
+        for (int h0 = (int)(it % chunks) * HPW; h0 < HT; h0 += chunks * HPW) {  // wave-uniform
+            const int hh = h0 + hw;
+            const bool is_q = hh < p.H, is_k = !is_q && hh < HK;
+            const int col0 = hh < HK ? hh * p.d : HK * p.d + (hh - HK) * p.dv;
+            const int64_t so = t * p.lds_ + col0;
+            f32x4 x = {0.f, 0.f, 0.f, 0.f}, y = {0.f, 0.f, 0.f, 0.f};
+            const bool qk = hh < HK && mine;
+            if (qk) {
+                x = ld4_dt(p.src, p.src_dt, so + a0);
+                if (p.bias) x += *(const f32x4*)(p.bias + col0 + a0);
+                if (LAYOUT && turns) {
+                    y = ld4_dt(p.src, p.src_dt, so + a1);
+                    if (p.bias) y += *(const f32x4*)(p.bias + col0 + a1);
+                }
+                if (is_k && p.tie_v) {  // the value is the key as it came
+                    const int64_t d0 = row + p.G * p.d + (hh - p.H) * p.dv;
+                    st4_dt(p.cache, p.c_dt, d0 + a0, x);
+                    if (LAYOUT && turns) st4_dt(p.cache, p.c_dt, d0 + a1, y);
+                }
+            }
+            const float* w = is_q ? p.qw : p.kw;
+            if (p.unit_norm || p.qw || p.kw) {
+                float ss = (x[0] * x[0] + x[1] * x[1]) + (x[2] * x[2] + x[3] * x[3]);
+                ss += (y[0] * y[0] + y[1] * y[1]) + (y[2] * y[2] + y[3] * y[3]);
+                for (int o = LPH >> 1; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
+                if (qk && (p.unit_norm || w)) {
+                    const float r = 1.0f / sqrtf(ss / (float)p.d + p.eps);
+                    x *= r, y *= r;
+                    if (w) {
+                        x *= *(const f32x4*)(w + a0);
+                        if (LAYOUT && turns) y *= *(const f32x4*)(w + a1);
+                    }
+                }
+            }
+            if (qk) {
+                if (turns) {
+                    if (LAYOUT) {
+#pragma unroll
+                        for (int e = 0; e < 4; ++e) {
+                            const float m = x[e], n = y[e];
+                            x[e] = m * c[e] - n * s[e];
+                            y[e] = n * c[e] + m * s[e];
+                        }
+                    } else {
+#pragma unroll
+                        for (int e = 0; e < 2; ++e) {
+                            const float m = x[2 * e], n = x[2 * e + 1];
+                            x[2 * e] = m * c[e] - n * s[e];
+                            x[2 * e + 1] = n * c[e] + m * s[e];
+                        }
+                    }
+                }
+                if (is_q) {
+                    const float sc = (p.qscale ? p.qscale[hh] : 1.0f) * qt;
+                    float* q = p.q_out + t * p.ldq + (int64_t)hh * p.d;
+                    *(f32x4*)(q + a0) = x * sc;
+                    if (LAYOUT && turns) *(f32x4*)(q + a1) = y * sc;
+                } else {
+                    const int64_t k0 = row + (int64_t)(hh - p.H) * p.d;
+                    st4_dt(p.cache, p.c_dt, k0 + a0, x);
+                    if (LAYOUT && turns) st4_dt(p.cache, p.c_dt, k0 + a1, y);
+                }
+            } else if (hh >= HK && hh < HT) {
+                const int64_t d0 = row + p.G * p.d + (int64_t)(hh - HK) * p.dv;
+                for (int i = 4 * u; i < p.dv; i += 4 * LPH) {
+                    f32x4 v = ld4_dt(p.src, p.src_dt, so + i);
+                    if (p.bias) v += *(const f32x4*)(p.bias + col0 + i);
+                    if (p.vmix) v = (1.0f - p.lam) * v + p.lam * *(const f32x4*)(p.vmix + t * p.ldvm + (hh - HK) * p.dv + i);
+                    st4_dt(p.cache, p.c_dt, d0 + i, v);
+                }
+            }
+        }
+    }
+}
+
 extern "C" int mi355_qkv_rows_append(int64_t tokens, int H, int G, int d, int dv, const void* src, int src_dt, int64_t ld_src, const float* bias, const float* qw,
                                      const float* kw, float eps, const float* qscale, int dims, int layout, const float* freq, const int* pos, const int* dst_row,
                                      float* q_out, int64_t ldq, void* cache, int c_dt, int64_t ldc, float qt_coef, int qt_every, const float* vmix, int64_t ldvm,
@@ -428,7 +527,19 @@ extern "C" int mi355_qkv_rows_append(int64_t tokens, int H, int G, int d, int dv
     p.lds_ = ld_src, p.ldq = ldq, p.ldc = ldc, p.src_dt = src_dt, p.c_dt = c_dt, p.H = H, p.G = G, p.GV = GV, p.d = d, p.dv = dv, p.dims = dims, p.layout = layout, p.eps = eps;
     p.vmix = vmix, p.ldvm = ldvm, p.lam = lam, p.qt_coef = qt_coef, p.qt_every = qt_every;
     p.unit_norm = unit_norm, p.rot_amp = rot_amp, p.tie_v = tie_v;
-    qkv_rows_kernel<<<rec_rows_grid(tokens * (H + G + GV), 4), 256, 0, ST(stream)>>>(tokens, p);
+    const int units = layout ? dims / 8 + (d - dims) / 4 : d / 4;
+    const bool vec = d % 4 == 0 && dv % 4 == 0 && dims % (layout ? 8 : 4) == 0 && units <= 64 && ld_src % 4 == 0 && ldq % 4 == 0 && ldc % 4 == 0 && ldvm % 4 == 0 && al16(src) &&
+                     al16(bias) && al16(qw) && al16(kw) && al16(q_out) && al16(cache) && al16(vmix);
+    if (vec) {
+        int lph = 1;
+        while (lph < units) lph *= 2;
+        const int passes = (H + G + (tie_v ? 0 : GV) + 64 / lph - 1) / (64 / lph), chunks = tokens < 2048 ? passes : 1;
+        const int grid = rec_rows_grid(tokens * chunks, 4);
+        if (layout) qkv_rows_vec_kernel<1><<<grid, 256, 0, ST(stream)>>>(tokens, p, lph, chunks);
+        else qkv_rows_vec_kernel<0><<<grid, 256, 0, ST(stream)>>>(tokens, p, lph, chunks);
+    } else {
+        qkv_rows_kernel<<<rec_rows_grid(tokens * (H + G + GV), 4), 256, 0, ST(stream)>>>(tokens, p);
+    }
     MI355_LAUNCH_CHECK("qkv_rows_append");
     return 0;
 }

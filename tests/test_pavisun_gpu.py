@@ -424,6 +424,37 @@ def test_table_experts_alone(dt, experts, top, ff):
     assert row_err(out.reshape(50, top, -1).sum(1) / top, want) < (3e-6 if dt == "float32" else 2e-2)
 
 
+@pytest.mark.parametrize("dt", DTYPES)
+@pytest.mark.parametrize("width,ff,experts,top", [(264, 520, 5, 2), (512, 300, 3, 1), (260, 256, 4, 3), (1024, 64, 9, 2)])
+def test_experts_of_every_number_of_rows(dt, width, ff, experts, top):
+    """From one token (the weights are streamed) to hundreds (tiles): one expert taking nearly every row, one taking none, widths that are multiples of 8 and not; a
+    token's rows do not depend on how many others there are, beyond rounding."""
+    from llm_quest_amd import kernels_seq as K
+    from llm_quest_amd.common.mixers import TableMoE
+
+    g = torch.Generator().manual_seed(width + ff)
+    r = lambda *s: (torch.randn(*s, generator=g) / s[-1] ** 0.5).to(BF16)
+    gates, ups, downs = [r(ff, width) for _ in range(experts)], [r(ff, width) for _ in range(experts)], [r(width, ff) for _ in range(experts)]
+    m = TableMoE(width, ff, experts, top, 1)
+    m.load_experts(gates, ups, downs)
+    m = m.to(DEV)
+    act = F32 if dt == "float32" else BF16
+    h = torch.randn(400, width, generator=g).to(act)
+    score = torch.rand(400, experts, generator=g) + torch.tensor([2.0 * (e == 1) - 5.0 * (e == 0 and top < experts) for e in range(experts)])
+    ids = score.argsort(dim=1, descending=True)[:, :top]
+    want = torch.empty(400, top, width, dtype=F64)
+    for e in range(experts):
+        z = h.double() @ gates[e].double().T
+        y = (z * torch.sigmoid(z) * (h.double() @ ups[e].double().T)) @ downs[e].double().T
+        want[ids == e] = y[(ids == e).any(1)]
+    for T in (1, 2, 33, 85, 130, 400):
+        offs, perm = K.moe_dispatch(ids[:T].reshape(-1).to(I32).to(DEV), experts)
+        wts = None if T % 2 else torch.rand(T, top, generator=g)
+        out = m.run_experts(h[:T].to(DEV), offs, perm, None if wts is None else wts.to(DEV)).reshape(T, top, width)
+        ref = want[:T] if wts is None else want[:T] * wts.double()[..., None]
+        assert float((out.cpu().double() - ref).abs().max()) < (2e-5 if dt == "float32" else 2e-2) * float(want.abs().max()), T
+
+
 def _cache_with_slot(cache):
     cache.open("s")
     return cache
